@@ -78,7 +78,9 @@ class ModelConfig:
     # routing: "softmax_topk" (mixtral: softmax→topk→renorm) |
     # "topk_softmax" (gpt-oss: topk logits→softmax over the k) |
     # "softmax_bias" (softmax over all experts; the choice adds a
-    # per-expert correction, the weights are the plain scores)
+    # per-expert correction and may be limited to the groups with the
+    # largest choice; the weights are the plain scores, renormalised with
+    # moe_norm_topk)
     moe_routing: str = "softmax_topk"
     # router logits in f32 (x and the router matrix are widened before the
     # product) instead of the activation dtype
@@ -103,6 +105,9 @@ class ModelConfig:
     # weights) to softmax_topk/topk_softmax
     moe_norm_topk: bool = True           # renormalize selected weights
     routed_scaling_factor: float = 1.0   # V3: 2.5
+    # router outputs beyond num_experts that hand the input through
+    # ("softmax_bias" routing); groups are formed over both
+    moe_identity_experts: int = 0
     n_group: int = 1                     # expert groups (V3: 8)
     topk_group: int = 1                  # groups kept per token (V3: 4)
     n_shared_experts: int = 0            # always-on experts (width = n*moe_ie)
@@ -145,6 +150,11 @@ class ModelConfig:
     # a run of layers executed several times with the same weights
     # (models/hybrid_config.py LoopSpec); None = every layer once
     layer_loop: Optional[object] = None
+    # hyper-connections: copies of the residual row a stack carries
+    # (0 = a single stream with plain residual sums)
+    residual_streams: int = 0
+    # factor of every sub-layer's output in the residual sum
+    residual_mult: float = 1.0
 
     @classmethod
     def from_hf_config(cls, cfg: dict, name: str = "") -> "ModelConfig":

@@ -1,6 +1,6 @@
 """Per-layer specifications for hybrid stacks (recurrent, windowed and
 latent attention layers mixed in one model) and the config.json readers of
-the Gurapel, Pokulorn, Munerax and Lokedra designs.
+the Gurapel, Pokulorn, Munerax, Lokedra and Vemenex designs.
 
 A homogeneous model is described by the flat ModelConfig fields; a hybrid
 one additionally carries `layer_specs`, one LayerSpec per layer, each
@@ -66,7 +66,10 @@ class MoESpec:
     groups are eligible; weights are the chosen scores times `scale`, not
     renormalised) or "softmax_bias" (softmax over all experts; the choice
     adds a per-expert correction to the scores, the weights are the chosen
-    scores without it, not renormalised). `act`: "silu_glu" (gated
+    scores without it, over their sum with `renorm`; with `groups` > 1 a
+    group scores its largest corrected score; the last `identity` router
+    outputs, beyond the `experts`, hand the input through and belong to
+    the groups like the others). `act`: "silu_glu" (gated
     experts), "relu2" (ungated, squared relu) or "clamped_glu"
     (g = min(gate, limit), u = clamp(up, ±limit), g·sigmoid(1.702 g)·
     (u + 1)). `shared_ff` > 0 adds an always-on expert of that width and
@@ -81,6 +84,8 @@ class MoESpec:
     scale: float = 1.0
     shared_ff: int = 0
     limit: float = 0.0            # clamp of "clamped_glu"
+    renorm: bool = False
+    identity: int = 0
 
 
 @dataclass(frozen=True)
@@ -90,7 +95,8 @@ class RotarySpec:
     2i + 1. With `factor` > 0 the frequencies are
     interpolated by parts (wavelengths beyond `original`/`slow` turns are
     divided by `factor`, those below `original`/`fast` turns kept, a
-    linear ramp between) and cos/sin are scaled by 0.1·ln(factor) + 1."""
+    linear ramp between) and cos/sin are scaled by 0.1·ln(factor) + 1.
+    `linear` divides every frequency (and leaves cos/sin as they are)."""
     dims: int
     base: float
     factor: float = 0.0          # 0 = plain rotation
@@ -98,12 +104,14 @@ class RotarySpec:
     fast: float = 32.0
     slow: float = 1.0
     interleaved: bool = False
+    linear: float = 1.0
 
     def frequencies(self):
         """(per-pair angular frequencies as a float64 list, magnitude)."""
         import math
         half = self.dims // 2
-        freq = [self.base ** (-2.0 * i / self.dims) for i in range(half)]
+        freq = [self.base ** (-2.0 * i / self.dims) / self.linear
+                for i in range(half)]
         if self.factor <= 0:
             return freq, 1.0
 
@@ -146,6 +154,12 @@ class RotaryAttnSpec:
     bias: bool = False            # biases on the q/k/v and output projections
     tied_values: bool = False     # no value projection: v = k as cached
     unit_sink: bool = False       # a sink of score 0: denominator 1 + sum
+    # q and k divided by their RMS per head after the rotation (no weight)
+    qk_unit_norm: bool = False
+    # a key's weight is sigmoid(score + a per-head bias): no softmax, no
+    # normalisation over the keys
+    sigmoid_scores: bool = False
+    head_gate: bool = False       # sigmoid output gate, one number per head
 
 
 @dataclass(frozen=True)
@@ -243,9 +257,11 @@ class LoopSpec:
 
 
 @dataclass(frozen=True)
-class GeluGLUSpec:
-    """Gated feed-forward down(gelu_tanh(gate)·up)."""
+class GLUSpec:
+    """Gated feed-forward down(act(gate)·up), act "gelu" (tanh form) or
+    "relu"."""
     ff: int
+    act: str = "gelu"
 
 
 @dataclass(frozen=True)
@@ -270,6 +286,8 @@ class LayerSpec:
     # Lokedra — "general_delta": DiagDeltaSpec; "latent_attention":
     # LatentAttnSpec; "parallel": RotaryAttnSpec beside HGRN2Spec, summed
     # with `branch_scales`; feed-forward `moe` or none.
+    # Vemenex — "attention" (sigmoid scores) and "attention_2" (unit sink,
+    # head gate): RotaryAttnSpec; feed-forward `glu`, `moe` or none.
     kind: str
     delta: Optional[DeltaRuleSpec] = None
     attn: Optional[WindowAttnSpec] = None
@@ -281,7 +299,7 @@ class LayerSpec:
     dense: Optional[DenseFFSpec] = None
     branch_scales: Tuple[float, float] = (1.0, 1.0)
     latent: Optional[LatentAttnSpec] = None
-    glu: Optional[GeluGLUSpec] = None
+    glu: Optional[GLUSpec] = None
     ddelta: Optional[DiagDeltaSpec] = None
     hgrn: Optional[HGRN2Spec] = None
 
@@ -367,7 +385,8 @@ def layer_moe_config(cfg: ModelConfig, moe: MoESpec) -> ModelConfig:
         moe_act="silu" if moe.act == "silu_glu" else moe.act,
         moe_bias=False, n_shared_experts=0,
         moe_shared_intermediate_size=moe.shared_ff, n_group=moe.groups,
-        topk_group=moe.keep_groups, moe_norm_topk=False,
+        topk_group=moe.keep_groups, moe_norm_topk=moe.renorm,
+        moe_identity_experts=moe.identity,
         routed_scaling_factor=moe.scale, moe_router_fp32=True,
         moe_act_limit=moe.limit)
 
@@ -462,12 +481,12 @@ def pokulorn_model_config(cfg: dict, name: str = "",
 # ---- Munerax ------------------------------------------------------------------
 
 def _munerax_ff(m):
-    """config `mlp` entry → (GeluGLUSpec | None, MoESpec | None)."""
+    """config `mlp` entry → (GLUSpec | None, MoESpec | None)."""
     if m is None:
         return None, None
     kind = m.get("kind", "dense")
     if kind == "dense":
-        return GeluGLUSpec(ff=int(m["ff"])), None
+        return GLUSpec(ff=int(m["ff"])), None
     if kind != "moe":
         raise ValueError(f"unsupported feed-forward kind {kind!r}")
     r = m["router"]
@@ -632,6 +651,84 @@ def lokedra_model_config(cfg: dict, name: str = "",
         rms_eps=float(cfg["norm"]["eps"]),
         embed_scale=float(cfg["embedding"].get("scale", 1.0)),
         rms_norm_offset=True, tie_word_embeddings=True, residual_fp32=True,
+        num_experts=moe.experts if moe else 0,
+        num_experts_per_tok=moe.top if moe else 0,
+        moe_intermediate_size=moe.ff if moe else 0, dtype=dtype)
+
+
+# ---- Vemenex ------------------------------------------------------------------
+
+def _vemenex_ff(m):
+    """config `mlp` entry → (GLUSpec | None, MoESpec | None)."""
+    if m is None:
+        return None, None
+    kind = m.get("kind", "dense")
+    if kind == "dense":
+        return GLUSpec(ff=int(m["ff"]), act="relu"), None
+    if kind != "moe":
+        raise ValueError(f"unsupported feed-forward kind {kind!r}")
+    r = m["router"]
+    g = r.get("groups") or {}
+    moe = MoESpec(
+        experts=int(r["experts"]), top=int(r["top"]),
+        ff=int(m["expert"]["ff"]), routing="softmax_bias",
+        act="clamped_glu", limit=float(m["expert"]["limit"]),
+        groups=int(g.get("count", 1)), keep_groups=int(g.get("keep", 1)),
+        renorm=True, identity=int(r.get("identity", 0)))
+    n = moe.experts + moe.identity
+    if n % moe.groups or not 1 <= moe.keep_groups <= moe.groups \
+            or moe.top > moe.keep_groups * (n // moe.groups):
+        raise ValueError(f"router: {n} outputs in {moe.groups} groups, "
+                         f"{moe.keep_groups} kept, top {moe.top}")
+    return None, moe
+
+
+def _vemenex_layer(entry: dict) -> LayerSpec:
+    kind, mx = entry["type"], entry["mixer"]
+    if kind not in ("attention", "attention_2"):
+        raise ValueError(f"unknown layer type {kind!r}")
+    sig = kind == "attention"
+    rot = None
+    if mx.get("rot"):
+        r = mx["rot"]
+        rot = RotarySpec(
+            dims=int(r["dims"]), base=float(r["base"]), interleaved=sig,
+            linear=float((r.get("scaling") or {}).get("factor", 1.0)))
+    glu, moe = _vemenex_ff(entry.get("mlp"))
+    return LayerSpec(kind, rattn=RotaryAttnSpec(
+        heads=int(mx["heads"]), kv_heads=int(mx["kv_heads"]),
+        dim=int(mx["dim"]), vdim=int(mx["vdim"]), scale=float(mx["scale"]),
+        rot=rot, window=int((mx.get("mask") or {}).get("size", 0)),
+        qk_norm=False, qk_unit_norm=True, sigmoid_scores=sig,
+        unit_sink=not sig, head_gate=not sig), glu=glu, moe=moe)
+
+
+def is_vemenex_config(cfg: dict) -> bool:
+    return cfg.get("architecture") == "Vemenex"
+
+
+def vemenex_model_config(cfg: dict, name: str = "",
+                         dtype: torch.dtype = torch.bfloat16) -> ModelConfig:
+    """config.json of a Vemenex checkpoint → ModelConfig (every size, the
+    layer order and every per-model constant come from the file). The
+    design has no position table, so its length limit is the engine's."""
+    specs: Tuple[LayerSpec, ...] = tuple(
+        _vemenex_layer(e) for e in cfg["layers"])
+    width = int(cfg["width"])
+    att = specs[0].rattn
+    moe = next((s.moe for s in specs if s.moe is not None), None)
+    glu = next((s.glu for s in specs if s.glu is not None), None)
+    return ModelConfig(
+        name=name or "vemenex", arch="vemenex", layer_specs=specs,
+        hidden_size=width, num_layers=len(specs),
+        num_heads=att.heads, num_kv_heads=att.kv_heads, head_dim=att.dim,
+        intermediate_size=glu.ff if glu else (moe.ff if moe else width),
+        vocab_size=int(cfg["vocab"]),
+        max_position=int(cfg.get("max_positions",
+                                 POKULORN_DEFAULT_MAX_POSITION)),
+        rms_eps=float(cfg["norm"]["eps"]),
+        residual_streams=int(cfg["streams"]),
+        residual_mult=float(cfg["residual_mult"]), residual_fp32=True,
         num_experts=moe.experts if moe else 0,
         num_experts_per_tok=moe.top if moe else 0,
         moe_intermediate_size=moe.ff if moe else 0, dtype=dtype)

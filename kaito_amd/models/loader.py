@@ -32,6 +32,8 @@ def load_safetensors_weights(model, path: str,
         return load_munerax_weights(model, path)
     if getattr(model.cfg, "arch", "llama") == "lokedra":
         return load_lokedra_weights(model, path)
+    if getattr(model.cfg, "arch", "llama") == "vemenex":
+        return load_vemenex_weights(model, path)
     from safetensors.torch import safe_open
 
     cfg = model.cfg
@@ -569,18 +571,69 @@ def load_lokedra_weights(model, path: str) -> None:
             continue
         fp = pre + "mlp."
         put(layer.scale_ff, get(pre + "ls2").float())
-        put(mlp.gate, get(fp + "router").float())
-        put(mlp.e_score_correction_bias, get(fp + "correction").float())
-        ie = mlp.ie_local
-        with torch.no_grad():
-            mlp.w_gate_up.zero_()
-            mlp.w_down.zero_()
-            for e in range(mlp.num_experts):
-                g, u, d = (get(f"{fp}e{e}.{n}") for n in ("gate", "up",
-                                                          "down"))
-                ff = g.shape[0]
-                dt = mlp.w_gate_up.dtype
-                mlp.w_gate_up[e, :ff].copy_(g.to(dt))
-                mlp.w_gate_up[e, ie:ie + ff].copy_(u.to(dt))
-                mlp.w_down[e, :, :ff].copy_(d.to(dt))
+        _load_routed(ck, mlp, fp)
+    ck.warn_unused()
+
+
+def _load_routed(ck, mlp, fp: str) -> None:
+    """Router, choice correction and gated experts under prefix fp (experts
+    zero-filled up to the kernels' tile width)."""
+    get, put = ck.get, ck.put
+    put(mlp.gate, get(fp + "router").float())
+    put(mlp.e_score_correction_bias, get(fp + "correction").float())
+    ie = mlp.ie_local
+    with torch.no_grad():
+        mlp.w_gate_up.zero_()
+        mlp.w_down.zero_()
+        for e in range(mlp.num_experts):
+            g, u, d = (get(f"{fp}e{e}.{n}") for n in ("gate", "up", "down"))
+            ff = g.shape[0]
+            dt = mlp.w_gate_up.dtype
+            mlp.w_gate_up[e, :ff].copy_(g.to(dt))
+            mlp.w_gate_up[e, ie:ie + ff].copy_(u.to(dt))
+            mlp.w_down[e, :, :ff].copy_(d.to(dt))
+
+
+def load_vemenex_weights(model, path: str) -> None:
+    """Vemenex checkpoint (flat tensor names, `l<i>.` per layer, mixer
+    tensors under `.mix.`, feed-forward under `.mlp.`, stream connections
+    under `.hc1.` / `.hc2.`, linear weights [out, in]) →
+    VemenexForCausalLM. Fuses each mixer's input projections, folds the
+    residual factor into the streams' write weights, stacks the experts and
+    widens norm weights, biases and connections to f32."""
+    ck = _FlatCheckpoint(path)
+    get, put = ck.get, ck.put
+
+    def one(name):                   # norm weights are a single number
+        return get(name).float().reshape(1)
+
+    put(model.embed_tokens.weight, get("embed"))
+    put(model.embed_norm, one("embed.norm"))
+    put(model.norm, one("final.norm").expand(model.norm.shape))
+    put(model.lm_head, get("head"))
+    for i, layer in enumerate(model.layers):
+        pre, mp, fp = f"l{i}.", f"l{i}.mix.", f"l{i}.mlp."
+        a, s = layer.attn, layer.attn.spec
+        for q, c in enumerate(layer.connections(), 1):
+            put(c.norm, one(f"{pre}norm{q}"))
+            put(c.w_in, get(f"{pre}hc{q}.in").float())
+            put(c.w_out, get(f"{pre}hc{q}.out").float()
+                * model.cfg.residual_mult)
+            put(c.mix, get(f"{pre}hc{q}.mix").float())
+        names = ("q", "k", "v") + (("g",) if s.head_gate else ())
+        w_in = torch.cat([get(mp + n) for n in names], 0)
+        if w_in.shape[0] != a.in_rows:
+            raise ValueError(f"{mp}: projection rows {w_in.shape[0]} vs "
+                             f"{a.in_rows} from the config")
+        put(a.qkv_proj, torch.nn.functional.pad(
+            w_in, (0, 0, 0, a.qkv_proj.shape[0] - a.in_rows)))
+        if s.sigmoid_scores:
+            put(a.score_bias, get(mp + "pb").float())
+        put(a.o_proj, get(mp + "o"))
+        if layer.spec.glu is not None:
+            put(layer.mlp.gate_up, torch.cat(
+                [get(fp + "gate"), get(fp + "up")], 0))
+            put(layer.mlp.down, get(fp + "down"))
+        elif layer.spec.moe is not None:
+            _load_routed(ck, layer.mlp, fp)
     ck.warn_unused()

@@ -3,7 +3,8 @@ recurrence, matrix-memory (mLSTM) recurrence, scalar-decay selective
 state space, softmax attention over the paged cache in two flavours
 (distance penalty without rotation; convolutions + rotation + window
 with kept first tokens or a chunked mask + sink, optionally with the
-keys as values), latent attention (one low-rank latent per token in the
+keys as values, optionally with sigmoid weights in place of the softmax
+and a gate per head), latent attention (one low-rank latent per token in the
 cache, optionally borrowed from an earlier layer, optionally with
 low-rank queries), the generalized delta rule with per-channel decay, and
 gated linear attention with a tied write gate (HGRN2). Each is a self-contained module parameterised by its spec
@@ -34,7 +35,7 @@ import torch.nn.functional as F
 
 from .. import ops
 from .hybrid_config import (DeltaRuleSpec, DenseFFSpec, DiagDeltaSpec,
-                            GeluGLUSpec, HGRN2Spec, LatentAttnSpec,
+                            GLUSpec, HGRN2Spec, LatentAttnSpec,
                             MLSTMSpec, RGLRUSpec, RotaryAttnSpec, SSDSpec,
                             WindowAttnSpec)
 
@@ -240,7 +241,9 @@ class RotaryWindowAttention(nn.Module):
     first value-mixing layer before they are cached, or be the keys
     themselves as cached (no value projection, one cache tensor); the
     projections may carry biases; the heads' outputs may be gated by
-    sigmoid of a fourth projection."""
+    sigmoid of a fourth projection, per value dimension or per head. The
+    norm of q and k may be a plain one behind the rotation, and a key's
+    weight may be sigmoid(score + a per-head bias) instead of a softmax."""
 
     def __init__(self, hidden: int, spec: RotaryAttnSpec, dtype,
                  norm_eps: float):
@@ -255,15 +258,20 @@ class RotaryWindowAttention(nn.Module):
         self.v_size = 0 if s.tied_values else s.kv_heads * s.vdim
         self.o_size = s.heads * s.vdim
         self.conv_ch = self.q_size + self.k_size + self.v_size
-        # fused input projection, rows [q | k | v | gate]
-        self.qkv_proj = _p(self.conv_ch + (self.o_size if s.gate else 0),
-                           hidden, dtype=dtype)
+        # fused input projection, rows [q | k | v | gate], padded so that
+        # the rows of its result stay 16-byte aligned
+        assert not (s.gate and s.head_gate)
+        self.in_rows = self.conv_ch + (self.o_size if s.gate else 0) \
+            + (s.heads if s.head_gate else 0)
+        self.qkv_proj = _p(-(-self.in_rows // 8) * 8 if s.head_gate
+                           else self.in_rows, hidden, dtype=dtype)
         self.qkv_bias = _p(self.qkv_proj.shape[0], dtype=dtype) \
             if s.bias else None
         self.o_bias = _p(hidden, dtype=dtype) if s.bias else None
         self.conv_weight = _p(self.conv_ch, s.conv_taps, dtype=torch.float32) \
             if s.conv_taps > 0 else None
         if s.qk_norm:
+            assert not s.qk_unit_norm
             self.q_norm = _p(s.dim, dtype=torch.float32)
             self.k_norm = _p(s.dim, dtype=torch.float32)
         else:
@@ -275,8 +283,10 @@ class RotaryWindowAttention(nn.Module):
                 freq, dtype=torch.float64).float(), persistent=False)
         else:
             self.inv_freq, self.rot_mag = None, 1.0
+        self.score_bias = _p(s.heads, dtype=torch.float32) \
+            if s.sigmoid_scores else None
         if s.unit_sink:
-            assert not s.sink
+            assert not s.sink and not s.sigmoid_scores
             self.register_buffer("sinks", torch.zeros(
                 s.heads, dtype=torch.float32), persistent=False)
         else:
@@ -335,7 +345,8 @@ class RotaryWindowAttention(nn.Module):
             q, k, v, self.q_norm, self.k_norm, self.norm_eps, cache["k"],
             v_cache, meta.slot_mapping, positions=positions,
             inv_freq=self.inv_freq, rot_mag=self.rot_mag, v_first=v_first,
-            v_lambda=lam)
+            v_lambda=lam, unit_norm=s.qk_unit_norm,
+            interleaved=s.rot is not None and s.rot.interleaved)
         tiles = None
         if meta.tile_seq is not None:
             tiles = (meta.tile_seq, meta.tile_qbase, meta.cu_seqlens,
@@ -344,7 +355,9 @@ class RotaryWindowAttention(nn.Module):
                                  meta.block_tables, meta.token_seq, positions,
                                  s.scale, window=s.window, tiles=tiles,
                                  keep_first=s.keep_first, sinks=self.sinks,
-                                 chunk=s.chunk)
+                                 chunk=s.chunk, sigmoid_bias=self.score_bias,
+                                 gate=p[:, self.conv_ch:self.in_rows]
+                                 if s.head_gate else None)
         o = o.reshape(T, self.o_size)
         if s.gate:
             o = ops.sigmoid_mul(o, p[:, self.conv_ch:])
@@ -610,17 +623,19 @@ class LatentAttention(nn.Module):
         return o[..., :V]
 
 
-class GeluGLU(nn.Module):
-    """Dense gated feed-forward down(gelu_tanh(gate x) · up x)."""
+class GatedFF(nn.Module):
+    """Dense gated feed-forward down(act(gate x) · up x), act gelu_tanh or
+    relu."""
 
-    def __init__(self, hidden: int, spec: GeluGLUSpec, dtype):
+    def __init__(self, hidden: int, spec: GLUSpec, dtype):
         super().__init__()
         self.spec = spec
+        self.act = {"gelu": ops.gelu_glu, "relu": ops.relu_glu}[spec.act]
         self.gate_up = _p(2 * spec.ff, hidden, dtype=dtype)   # [gate | up]
         self.down = _p(hidden, spec.ff, dtype=dtype)
 
     def forward(self, x):
-        return F.linear(ops.gelu_glu(F.linear(x, self.gate_up)), self.down)
+        return F.linear(self.act(F.linear(x, self.gate_up)), self.down)
 
 
 class DiagDeltaMixer(nn.Module):

@@ -40,6 +40,9 @@ class MoEMLP(nn.Module):
         e = cfg.num_experts
         self.top_k = cfg.num_experts_per_tok
         self.num_experts = e
+        # router outputs: the experts, then those that hand x through
+        self.n_identity = cfg.moe_identity_experts
+        self.n_route = e + self.n_identity
         if tp > 1 and e % tp == 0:
             # expert parallelism: contiguous expert slice per rank
             self.e_local = e // tp
@@ -54,8 +57,9 @@ class MoEMLP(nn.Module):
         # before the product, so no logit is rounded to the activation
         # dtype before top-k
         self.gate = nn.Parameter(
-            torch.empty(e, h, dtype=torch.float32 if cfg.moe_router_fp32
-                        else cfg.dtype), requires_grad=False)
+            torch.empty(self.n_route, h, dtype=torch.float32
+                        if cfg.moe_router_fp32 else cfg.dtype),
+            requires_grad=False)
         # "relu2": ungated experts down(relu(up x)^2); everything else is
         # gated (act(gate x) * up x)
         self.gated = cfg.moe_act != "relu2"
@@ -87,7 +91,12 @@ class MoEMLP(nn.Module):
         # per-expert selection bias (deepseek-v3 noaux_tc; softmax_bias)
         if cfg.moe_routing in ("noaux_tc", "softmax_bias"):
             self.e_score_correction_bias = nn.Parameter(
-                torch.empty(e, dtype=torch.float32), requires_grad=False)
+                torch.empty(self.n_route, dtype=torch.float32),
+                requires_grad=False)
+        if self.n_identity:
+            if cfg.moe_routing != "softmax_bias" or tp > 1:
+                raise NotImplementedError(
+                    "identity experts: softmax_bias routing, one rank")
         # deepseek shared experts: always-on dense SwiGLU of width
         # n_shared * moe_ie, IE-sharded over TP; its down output is a
         # TP-partial like the routed output, so both ride ONE all-reduce
@@ -107,7 +116,8 @@ class MoEMLP(nn.Module):
 
     def _route(self, x: torch.Tensor):
         """Device-only top-k routing + expert sort. Returns
-        (sorted_tok int32 [TK], gates f32 [TK], offsets int32 [E+1])."""
+        (sorted_tok int32 [TK], gates f32 [TK], offsets int32 [E+1],
+        weight f32 [T] on identity experts or None)."""
         T = x.size(0)
         cfg = self.cfg
         if cfg.moe_router_fp32:
@@ -137,12 +147,15 @@ class MoEMLP(nn.Module):
                 topw = topw / (topw.sum(-1, keepdim=True) + 1e-20)
             topw = topw * cfg.routed_scaling_factor
         elif cfg.moe_routing == "softmax_bias":
-            # softmax over all experts; the choice adds the correction,
-            # the weights are the chosen scores themselves
-            scores = torch.softmax(logits.float(), dim=-1)
-            topi = (scores + self.e_score_correction_bias).topk(
-                self.top_k, dim=-1)[1]
-            topw = scores.gather(1, topi)
+            # softmax over all outputs; the choice adds the correction
+            # (and is group-limited), the weights are the chosen scores
+            topi, topw, w_id = ops.moe_route(
+                logits.float(), self.e_score_correction_bias, self.top_k,
+                self.num_experts, cfg.n_group, cfg.topk_group,
+                cfg.moe_norm_topk, cfg.routed_scaling_factor)
+            # identity outputs sort behind every expert's rows
+            return ops.moe_sort(topi, topw, self.n_route) \
+                + (w_id if self.n_identity else None,)
         elif cfg.moe_routing == "topk_softmax":
             # gpt-oss: top-k on raw logits, softmax over the selected k
             topl, topi = torch.topk(logits.float(), self.top_k, dim=-1)
@@ -166,7 +179,7 @@ class MoEMLP(nn.Module):
         offsets = torch.zeros(self.num_experts + 1, device=x.device,
                               dtype=torch.int32)
         torch.cumsum(counts, 0, out=offsets[1:])
-        return sorted_tok, gates, offsets
+        return sorted_tok, gates, offsets, None
 
     # fused kernels win at decode-sized batches (weight-streaming
     # bound, graph-capturable); per-expert hipBLASLt GEMMs win at
@@ -179,9 +192,14 @@ class MoEMLP(nn.Module):
     import os as _os
     FUSED_MAX_TOKENS = int(_os.environ.get("KAITO_MOE_FUSED_MAX", "4096"))
 
-    def forward(self, x: torch.Tensor) -> torch.Tensor:
+    def forward(self, x: torch.Tensor,
+                keep_f32: bool = False) -> torch.Tensor:
+        """keep_f32: the routed sum is returned as accumulated, in f32."""
         T, H = x.shape
-        sorted_tok, gates, offsets = self._route(x)
+        sorted_tok, gates, offsets, w_id = self._route(x)
+        # the routed sum starts from the identity experts' share
+        out32 = torch.zeros(T, H, dtype=torch.float32, device=x.device) \
+            if w_id is None else x * w_id[:, None]
         fused_shapes = (x.is_cuda and x.dtype == torch.bfloat16
                         and H % 64 == 0 and self.ie_local % 64 == 0)
         # under hipGraph capture the fused kernels are mandatory (the
@@ -190,9 +208,10 @@ class MoEMLP(nn.Module):
         # at bs=768 (profiles/r02_perf_notes.md)
         if fused_shapes and (T * self.top_k <= self.FUSED_MAX_TOKENS
                              or torch.cuda.is_current_stream_capturing()):
-            out = self._forward_fused(x, sorted_tok, gates, offsets)
+            self._forward_fused(x, sorted_tok, gates, offsets, out32)
         else:
-            out = self._forward_loop(x, sorted_tok, gates, offsets)
+            self._forward_loop(x, sorted_tok, gates, offsets, out32)
+        out = out32 if keep_f32 else out32.to(x.dtype)
         if self.w_shared_gate_up is not None:   # deepseek shared experts
             h1 = torch.nn.functional.linear(x, self.w_shared_gate_up)
             out = out + torch.nn.functional.linear(
@@ -202,8 +221,9 @@ class MoEMLP(nn.Module):
             out = tp_all_reduce(out)
         return out
 
-    def _forward_fused(self, x, sorted_tok, gates, offsets):
-        """Static-shape HIP grouped GEMMs (graph-capturable)."""
+    def _forward_fused(self, x, sorted_tok, gates, offsets, out32):
+        """Static-shape HIP grouped GEMMs (graph-capturable), added into
+        out32."""
         T, H = x.shape
         TK = T * self.top_k
         # staging reads WHOLE 64-row tiles from unaligned expert offsets:
@@ -214,18 +234,14 @@ class MoEMLP(nn.Module):
         ops.moe_gate_silu(act, x, self.w_gate_up, sorted_tok, offsets,
                           self.e_base, self.e_local, self.b_gate_up,
                           self.act_mode, self.act_limit)
-        out32 = torch.zeros(T, H, dtype=torch.float32, device=x.device)
         ops.moe_down_scatter(out32, act, self.w_down, sorted_tok, gates,
                              offsets, self.e_base, self.e_local,
                              self.b_down)
-        return out32.to(x.dtype)
 
-    def _forward_loop(self, x, sorted_tok, gates, offsets):
+    def _forward_loop(self, x, sorted_tok, gates, offsets, out):
         """Per-expert torch GEMMs (CPU tests / odd shapes). Host sync on
         the segment sizes — never used on the GPU hot path."""
         off = offsets.tolist()
-        # f32 accumulation over a token's experts, like the fused path
-        out = torch.zeros(x.shape, dtype=torch.float32, device=x.device)
         idx64 = sorted_tok.long()
         for le in range(self.e_local):
             e = self.e_base + le
@@ -246,5 +262,5 @@ class MoEMLP(nn.Module):
             y = torch.nn.functional.linear(
                 act, self.w_down[le],
                 self.b_down[le] if self.b_down is not None else None)
+            # f32 accumulation over a token's experts, like the fused path
             out.index_add_(0, rows, y.float() * gates[s:t, None])
-        return out.to(x.dtype)

@@ -7,7 +7,7 @@ f32; sub-layers see its norm rounded to the activation dtype. The mixer
 is LatentAttention (models/mixers.py): the paged cache holds one
 low-rank latent and one rotated key part per token; a layer may read an
 earlier layer's cache instead of projecting its own. The feed-forward is
-GeluGLU or the engine's MoEMLP with squared-relu experts, group-limited
+GatedFF or the engine's MoEMLP with squared-relu experts, group-limited
 sigmoid routing and an always-on shared expert.
 
 Input: the scaled token embedding plus a hashed bigram embedding; the
@@ -31,7 +31,7 @@ from .. import ops
 from ..engine.config import ModelConfig
 from .hybrid_base import HybridStackBase, MixerLayerBase, f32_vector
 from .hybrid_config import LayerSpec, layer_moe_config
-from .mixers import GeluGLU, LatentAttention
+from .mixers import GatedFF, LatentAttention
 from .moe import MoEMLP
 
 
@@ -45,7 +45,7 @@ class MuneraxLayer(MixerLayerBase):
         self.attn = LatentAttention(h, spec.latent, dt, eps)
         self.norm1 = f32_vector(h)
         if spec.glu is not None:
-            self.mlp = GeluGLU(h, spec.glu, dt)
+            self.mlp = GatedFF(h, spec.glu, dt)
         elif spec.moe is not None:
             self.mlp = MoEMLP(layer_moe_config(cfg, spec.moe))
         else:

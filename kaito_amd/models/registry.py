@@ -27,6 +27,7 @@ MODEL_CLASSES: Dict[str, str] = {
     "pokulorn": "kaito_amd.models.pokulorn:PokulornForCausalLM",
     "munerax": "kaito_amd.models.munerax:MuneraxForCausalLM",
     "lokedra": "kaito_amd.models.lokedra:LokedraForCausalLM",
+    "vemenex": "kaito_amd.models.vemenex:VemenexForCausalLM",
 }
 
 
@@ -46,8 +47,9 @@ def config_from_checkpoint(cfg_json: dict, name: str = "",
     own architecture tag."""
     from .hybrid_config import (gurapel_model_config, is_gurapel_config,
                                 is_lokedra_config, is_munerax_config,
-                                is_pokulorn_config, lokedra_model_config,
-                                munerax_model_config, pokulorn_model_config)
+                                is_pokulorn_config, is_vemenex_config,
+                                lokedra_model_config, munerax_model_config,
+                                pokulorn_model_config, vemenex_model_config)
     kw = {"dtype": dtype} if dtype is not None else {}
     if is_gurapel_config(cfg_json):
         return gurapel_model_config(cfg_json, name=name, **kw)
@@ -57,6 +59,8 @@ def config_from_checkpoint(cfg_json: dict, name: str = "",
         return munerax_model_config(cfg_json, name=name, **kw)
     if is_lokedra_config(cfg_json):
         return lokedra_model_config(cfg_json, name=name, **kw)
+    if is_vemenex_config(cfg_json):
+        return vemenex_model_config(cfg_json, name=name, **kw)
     cfg = ModelConfig.from_hf_config(cfg_json, name=name)
     if dtype is not None:
         import dataclasses
@@ -476,3 +480,37 @@ def _tiny_lokedra() -> ModelConfig:
 
 
 register(_tiny_lokedra())
+
+
+def _tiny_vemenex() -> ModelConfig:
+    """A small hyper-connected stack (sigmoid-weight attention, gated
+    attention with a unit sink, dense and routed feed-forwards with
+    identity experts) for tests and smoke runs (random weights)."""
+    from .hybrid_config import vemenex_model_config
+
+    def mixer(**kw):
+        m = {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 24,
+             "mask": {"size": 40}, "scale": 0.25,
+             "rot": {"base": 10000.0, "dims": 16}}
+        m.update(kw)
+        return m
+    moe = {"kind": "moe", "expert": {"ff": 48, "limit": 2.0},
+           "router": {"experts": 7, "identity": 2, "top": 2,
+                      "groups": {"count": 3, "keep": 2}}}
+    layers = [
+        {"type": "attention_2", "mixer": mixer(), "mlp": moe},
+        {"type": "attention", "mixer": mixer(
+            heads=3, kv_heads=3, mask={"size": 25},
+            rot={"base": 5000.0, "dims": 8, "scaling": {"factor": 2.0}}),
+         "mlp": {"kind": "dense", "ff": 224}},
+        {"type": "attention", "mixer": mixer(rot={
+            "base": 10000.0, "dims": 16, "scaling": {"factor": 3.0}}),
+         "mlp": None},
+    ]
+    return vemenex_model_config({
+        "architecture": "Vemenex", "layers": layers, "norm": {"eps": 1e-5},
+        "residual_mult": 0.6, "streams": 2, "vocab": 512, "width": 192,
+        "max_positions": 1024}, name="tiny-vemenex-test")
+
+
+register(_tiny_vemenex())

@@ -29,6 +29,7 @@ for _g, _names in {
              "context_attention mfma_tile_gemm paged_read_bw"),
     "mla": "mla_decode mla_cache_write",
     "moe": "moe_gate_silu moe_down_scatter",
+    "route": "moe_route moe_sort",
     "quant": "w4a16_gemv w4a16_dequant w4a16_gemm lora_shrink lora_expand",
     "comm": ("allreduce_rmsnorm one_shot_ar_rmsnorm ipc_handle ipc_open "
              "ipc_close"),
@@ -36,12 +37,13 @@ for _g, _names in {
             "qk_norm_cache_write window_attention window_attention_tiles "
             "post_norm_residual rms_norm_cast residual_add_norm "
             "scaled_residual_add_norm token_shift "
-            "clamped_glu sigmoid_mul gelu_glu relu2"),
+            "clamped_glu sigmoid_mul gelu_glu relu_glu relu2"),
     "latent": ("bigram_embed latent_rope_cache_write latent_attention "
                "latent_expand"),
     "delta": "gated_delta_rule rglru_scan",
     "diag": "diag_delta_rule hgrn2_scan",
     "decay": "mlstm_scan ssd_scan",
+    "streams": "stream_mix_norm stream_embed",
 }.items():
     for _n in _names.split():
         _OP_GROUP[_n] = _g
@@ -329,6 +331,43 @@ def moe_down_scatter(out: torch.Tensor, act: torch.Tensor,
                                      offsets, b, e_base, n_local_experts)
 
 
+MOE_ROUTE_MAX = (1024, 64, 64)      # router outputs, chosen, groups
+
+
+def moe_route(logits, correction, top: int, n_real: int, groups: int = 1,
+              keep: int = 1, renorm: bool = False, scale: float = 1.0):
+    """Expert choice from f32 router logits [T, N]: scores s = softmax; the
+    choice adds `correction` [N] f32; outputs form `groups` equal groups of
+    neighbours scored by their largest choice, of which the `keep` best
+    stay eligible; the `top` largest eligible choices are taken. Weights
+    are s (without the correction), over their sum + 1e-20 with `renorm`,
+    times scale. Returns (indices [T, top] int32, weights [T, top] f32,
+    summed weight [T] f32 of the taken outputs with index >= n_real)."""
+    if logits.is_cuda:
+        T = logits.size(0)
+        f32 = dict(dtype=torch.float32, device=logits.device)
+        topi = torch.empty(T, top, dtype=torch.int32, device=logits.device)
+        topw, w_id = torch.empty(T, top, **f32), torch.empty(T, **f32)
+        _K.moe_route(topi, topw, w_id, logits, correction, n_real, groups,
+                     keep, renorm, scale)
+        return topi, topw, w_id
+    return torch_ref.moe_route(logits, correction, top, n_real, groups, keep,
+                               renorm, scale)
+
+
+def moe_sort(topi, topw, n: int):
+    """(token, expert) pairs ordered by expert: (token of each sorted row
+    [TK] int32, its weight [TK] f32, exclusive offsets [n + 1] int32)."""
+    if topi.is_cuda:
+        TK, dev = topi.numel(), topi.device
+        tok = torch.empty(TK, dtype=torch.int32, device=dev)
+        gates = torch.empty(TK, dtype=torch.float32, device=dev)
+        offsets = torch.empty(n + 1, dtype=torch.int32, device=dev)
+        _K.moe_sort(tok, gates, offsets, topi, topw)
+        return tok, gates, offsets
+    return torch_ref.moe_sort(topi, topw, n)
+
+
 def w4a16_gemv(x: torch.Tensor, qweight: torch.Tensor, scales: torch.Tensor,
                zeros: torch.Tensor, group: int) -> torch.Tensor:
     """Group-quantized W4A16 linear, small M (decode): out = x @ W^T with
@@ -441,14 +480,17 @@ def rglru_scan(u, gates, y, decay_rate, state, cu_seqlens, state_slots,
 def qk_norm_cache_write(q, k, v, q_w, k_w, eps: float, k_cache, v_cache,
                         slot_mapping, positions=None, inv_freq=None,
                         rot_mag: float = 1.0, v_first=None,
-                        v_lambda: float = 0.0):
+                        v_lambda: float = 0.0, unit_norm: bool = False,
+                        interleaved: bool = False):
     """Per-head RMS norm of q [T, H, D] / k [T, G, D] (f32 weights [D] or
     None), optional rotation (inv_freq [R] f32: dim i of every head is
-    paired with dim i + R, angle = position * inv_freq[i] in f32, cos and
+    paired with dim i + R, or with `interleaved` dim 2i with 2i + 1,
+    angle = position * inv_freq[i] in f32, cos and
     sin times rot_mag), optional value blend v <- (1 - v_lambda) v +
     v_lambda v_first, fused with the scatter of k and v [T, G, V] into
-    the paged caches [blocks, G, block_size, D|V]. Returns q normed and
-    rotated, [T, H, D]."""
+    the paged caches [blocks, G, block_size, D|V]. With `unit_norm` (and
+    no weights) q and k are divided by their RMS per head after the
+    rotation. Returns q normed and rotated, [T, H, D]."""
     if q.is_cuda:
         qn = torch.empty(q.shape, dtype=q.dtype, device=q.device)
         rot = inv_freq is not None and inv_freq.numel() > 0
@@ -459,11 +501,13 @@ def qk_norm_cache_write(q, k, v, q_w, k_w, eps: float, k_cache, v_cache,
                                               device=q.device),
             inv_freq if rot else _none(None, q), rot_mag,
             v_first if v_first is not None else
-            torch.empty(0, dtype=q.dtype, device=q.device), v_lambda)
+            torch.empty(0, dtype=q.dtype, device=q.device), v_lambda,
+            unit_norm, interleaved)
         return qn
     return torch_ref.qk_norm_cache_write(q, k, v, q_w, k_w, eps, k_cache,
                                          v_cache, slot_mapping, positions,
-                                         inv_freq, rot_mag, v_first, v_lambda)
+                                         inv_freq, rot_mag, v_first, v_lambda,
+                                         unit_norm, interleaved)
 
 
 WINDOW_MFMA_SIZES = (64, 128, 256)          # key sizes of the MFMA kernel
@@ -473,14 +517,19 @@ WINDOW_MFMA_VSIZES = (32, 64, 128, 256)     # value sizes
 def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
                      scale: float, softcap: float = 0.0, r1=None, r2=None,
                      window: int = 0, tiles=None, keep_first: int = 0,
-                     sinks=None, chunk: int = 0):
+                     sinks=None, chunk: int = 0, sigmoid_bias=None,
+                     gate=None):
     """Causal attention of query rows [T, H, D] over the paged cache (key
     size D, value size V may differ). A query at position i sees keys
     j <= i with i - j < window or j < keep_first (window <= 0: all), or,
     with `chunk` > 0, keys j <= i of i's own block of `chunk` absolute
     positions (block b = positions [b*chunk, (b+1)*chunk)). Options: tanh score capping, the distance penalty
     r1*ln(1 + r2*distance), and per-head `sinks` [H] f32 whose exp joins
-    the softmax denominator. Returns [T, H, V].
+    the softmax denominator. With
+    `sigmoid_bias` [H] f32 there is no softmax: a visible key's weight is
+    sigmoid(score + bias), not normalised over the keys. `gate` [T, H]
+    (row stride free) multiplies every head's output by its sigmoid.
+    Returns [T, H, V].
 
     `tiles` = (tile_seq, tile_qbase, cu_seqlens, seq_starts) describes the
     step's chunks as 64-row query tiles (build_query_tiles); with it, bf16
@@ -498,17 +547,19 @@ def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
             _K.window_attention_tiles(
                 out, q, k_cache, v_cache, block_tables, tile_seq, tile_qbase,
                 cu, starts, scale, softcap, _none(r1, q), _none(r2, q),
-                window, keep_first, _none(sinks, q), chunk)
+                window, keep_first, _none(sinks, q), chunk,
+                _none(sigmoid_bias, q), _none(gate, q))
             return out
         _K.window_attention(out, q, k_cache, v_cache, block_tables, token_seq,
                             positions, scale, softcap, _none(r1, q),
                             _none(r2, q), window, keep_first,
-                            _none(sinks, q), chunk)
+                            _none(sinks, q), chunk, _none(sigmoid_bias, q),
+                            _none(gate, q))
         return out
     return torch_ref.window_attention(q, k_cache, v_cache, block_tables,
                                       token_seq, positions, scale, softcap,
                                       r1, r2, window, keep_first, sinks,
-                                      chunk)
+                                      chunk, sigmoid_bias, gate)
 
 
 def build_query_tiles(chunk_lens, device):
@@ -632,6 +683,16 @@ def gelu_glu(gu):
         _K.gelu_glu(out, gu)
         return out
     return torch_ref.gelu_glu(gu)
+
+
+def relu_glu(gu):
+    """[gate | up] rows [T, 2F] -> relu(gate) * up [T, F]."""
+    if gu.is_cuda:
+        out = torch.empty(gu.size(0), gu.size(1) // 2, dtype=gu.dtype,
+                          device=gu.device)
+        _K.relu_glu(out, gu)
+        return out
+    return torch_ref.relu_glu(gu)
 
 
 def relu2(x):
@@ -858,3 +919,38 @@ def hgrn2_scan(q, v, f_pre, lower, norm_w, state, cu_seqlens, state_slots,
     return torch_ref.hgrn2_scan(q, v, f_pre, lower, norm_w, state,
                                 cu_seqlens, state_slots, seq_starts,
                                 norm_eps)
+
+
+# ---- hyper-connected residual streams (kernel group "streams") -------------
+
+def stream_embed(ids, table, g, w_in, w, eps: float):
+    """Opens a stack of S residual streams (S = len(w_in)): RMS-normed table
+    rows times g as S equal f32 copies [T, S, H], and the first sub-layer's
+    input rms(sum_s w_in[s] x_s)*w in the table's dtype. g and w are f32,
+    one number or one per coordinate. Returns (x, h)."""
+    if ids.is_cuda:
+        T, H = ids.numel(), table.size(1)
+        x = torch.empty(T, w_in.numel(), H, dtype=torch.float32,
+                        device=ids.device)
+        h = torch.empty(T, H, dtype=table.dtype, device=ids.device)
+        _K.stream_embed(x, h, ids, table, g, w_in, w, eps)
+        return x, h
+    return torch_ref.stream_embed(ids, table, g, w_in, w, eps)
+
+
+def stream_mix_norm(x, y, mix, w_out, w_in, w, eps: float, out_dtype,
+                    write_x: bool = True):
+    """A sub-layer's write and the next one's read on residual streams x
+    [T, S, H] f32: x_t <- sum_s mix[s, t] x_s + w_out[t]*y for all t from
+    the old streams, in place; u = sum_s w_in[s] x_s of the new ones.
+    Returns rms(u)*w in out_dtype, or u itself with w None (then
+    write_x=False leaves the streams unstored). y [T, H] may be the
+    activation dtype or f32; w is one number or one per coordinate."""
+    if x.is_cuda:
+        h = torch.empty(x.size(0), x.size(2), dtype=out_dtype,
+                        device=x.device)
+        _K.stream_mix_norm(x, h, y, mix, w_out, w_in, _none(w, x), eps,
+                           write_x)
+        return h
+    return torch_ref.stream_mix_norm(x, y, mix, w_out, w_in, w, eps,
+                                     out_dtype, write_x)

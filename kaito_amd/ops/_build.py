@@ -34,6 +34,8 @@ GROUPS: Dict[str, List[str]] = {
              "context_attention.hip", "diag.hip", "mfma_probe.hip"],
     "mla": ["bind_mla.cpp", "mla_attention.hip"],
     "moe": ["bind_moe.cpp", "moe.hip"],
+    # expert choice (softmax, correction, groups, top-k) and expert sort
+    "route": ["moe_route.hip"],
     "quant": ["bind_quant.cpp", "w4a16.hip", "lora.hip"],
     "comm": ["bind_comm.cpp", "allreduce_rmsnorm.hip"],
     # hybrid stacks (each source registers its own ops). "mix": what every
@@ -50,6 +52,8 @@ GROUPS: Dict[str, List[str]] = {
     # matrix recurrences with a decay per state row: generalized delta
     # rule, gated linear attention with a tied write gate
     "diag": ["diag_delta.hip"],
+    # hyper-connected residual streams
+    "streams": ["streams.hip"],
 }
 
 

@@ -6,6 +6,7 @@
 //   sigmoid_mul:  x * sigmoid(gate); a gate row narrower than x serves
 //                 groups of adjacent columns (one gate per head)
 //   gelu_glu:     [gate | up] rows [T, 2F] -> gelu_tanh(gate) * up
+//   relu_glu:     [gate | up] rows [T, 2F] -> relu(gate) * up
 //   relu2:        relu(x)^2
 #include "mix_common.h"
 
@@ -68,7 +69,14 @@ __global__ void sigmoid_mul_kernel(T* __restrict__ out,
              sigmoid_f(act_ld(gate + (int64_t)t * g_s0 + i / rep)));
 }
 
-// mode 0: gelu_tanh(in[i]) * in[F + i]; mode 1: relu(in[i])^2
+// mode 0: gelu_tanh(in[i]) * in[F + i]; mode 1: relu(in[i])^2; mode 2:
+// relu(in[i]) * in[F + i]
+KAITO_DEV float unary_glu_f(const int mode, const float a, const float b) {
+  if (mode == 0) return gelu_tanh_f(a) * b;
+  const float m = fmaxf(a, 0.f);
+  return mode == 1 ? m * m : m * b;
+}
+
 template <typename T>
 __global__ void unary_glu_kernel(T* __restrict__ out, const T* __restrict__ in,
                                  const int64_t in_s0, const int F,
@@ -77,11 +85,8 @@ __global__ void unary_glu_kernel(T* __restrict__ out, const T* __restrict__ in,
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= F) return;
   const T* row = in + (int64_t)t * in_s0;
-  const float a = act_ld(row + i);
-  float r;
-  if (mode == 0) r = gelu_tanh_f(a) * act_ld(row + F + i);
-  else { const float m = fmaxf(a, 0.f); r = m * m; }
-  act_st(out + (int64_t)t * F + i, r);
+  const float b = mode == 1 ? 0.0f : act_ld(row + F + i);
+  act_st(out + (int64_t)t * F + i, unary_glu_f(mode, act_ld(row + i), b));
 }
 
 template <typename T>
@@ -97,17 +102,13 @@ __global__ void unary_glu_vec_kernel(T* __restrict__ out,
   T av[VEC], bv[VEC], ov[VEC];
   *reinterpret_cast<float4_t*>(av) =
       *reinterpret_cast<const float4_t*>(row + i);
-  if (mode == 0)
+  *reinterpret_cast<float4_t*>(bv) = float4_t{0.f, 0.f, 0.f, 0.f};
+  if (mode != 1)
     *reinterpret_cast<float4_t*>(bv) =
         *reinterpret_cast<const float4_t*>(row + F + i);
 #pragma unroll
-  for (int e = 0; e < VEC; e++) {
-    const float a = act_ld(av + e);
-    float r;
-    if (mode == 0) r = gelu_tanh_f(a) * act_ld(bv + e);
-    else { const float m = fmaxf(a, 0.f); r = m * m; }
-    act_st(ov + e, r);
-  }
+  for (int e = 0; e < VEC; e++)
+    act_st(ov + e, unary_glu_f(mode, act_ld(av + e), act_ld(bv + e)));
   *reinterpret_cast<float4_t*>(out + (int64_t)t * F + i) =
       *reinterpret_cast<const float4_t*>(ov);
 }
@@ -212,6 +213,11 @@ void gelu_glu(at::Tensor out, at::Tensor gu) {
   unary_glu(out, gu, gu.size(1) / 2, 0);
 }
 
+void relu_glu(at::Tensor out, at::Tensor gu) {
+  TORCH_CHECK(gu.dim() == 2 && gu.size(1) % 2 == 0);
+  unary_glu(out, gu, gu.size(1) / 2, 2);
+}
+
 void relu2(at::Tensor out, at::Tensor x) {
   TORCH_CHECK(x.dim() == 2);
   unary_glu(out, x, x.size(1), 1);
@@ -223,11 +229,13 @@ TORCH_LIBRARY_FRAGMENT(kaito, m) {
   m.def("clamped_glu(Tensor(a!) out, Tensor gu, float limit, float alpha) -> ()");
   m.def("sigmoid_mul(Tensor(a!) out, Tensor x, Tensor gate) -> ()");
   m.def("gelu_glu(Tensor(a!) out, Tensor gu) -> ()");
+  m.def("relu_glu(Tensor(a!) out, Tensor gu) -> ()");
   m.def("relu2(Tensor(a!) out, Tensor x) -> ()");
 }
 TORCH_LIBRARY_IMPL(kaito, CUDA, m) {
   m.impl("clamped_glu", &kaito::clamped_glu);
   m.impl("sigmoid_mul", &kaito::sigmoid_mul);
   m.impl("gelu_glu", &kaito::gelu_glu);
+  m.impl("relu_glu", &kaito::relu_glu);
   m.impl("relu2", &kaito::relu2);
 }

@@ -11,10 +11,18 @@
 //   sinks:        with sink_h given, exp(sink_h) joins the softmax
 //                 denominator (no key, no value): the running maximum
 //                 starts at sink_h and the running sum at 1
+//   sigmoid:      with a per-head bias pb given there is no softmax: the
+//                 weight of a visible key is sigmoid(score + pb_h), and
+//                 the weights are not normalised over the keys
+//   gate:         with a pre-activation gate[t, h] given, the head's
+//                 output is multiplied by its sigmoid
 //
 // The q/k norm kernel optionally rotates the first 2R dims of every head
-// (dim i paired with i + R, angle = position * inv_freq[i], all f32) and
-// blends v with another layer's values before the cache write.
+// (dim i paired with i + R, or 2i with 2i + 1; angle = position *
+// inv_freq[i], all f32) and blends v with another layer's values before
+// the cache write. The norm is a weighted RMS norm ahead of the rotation or
+// a plain one behind it; a rotation keeps a row's sum of squares, so the
+// plain one also takes its statistic from the row as loaded.
 //
 // Key size D and value size V are independent; caches are
 // [blocks, G, block_size, D|V] in the activation dtype. Scores, softmax
@@ -40,31 +48,33 @@ namespace {
 // grid (T, H + 2G): blockIdx.y < H → q head; < H+G → k head; else v head.
 template <typename T>
 KAITO_DEV void norm_rotate_row(T* __restrict__ dst, const T* __restrict__ src,
-                               const float* __restrict__ w, const float eps,
+                               const float* __restrict__ w,
+                               const bool unit_norm, const float eps,
                                const int D, const float* __restrict__ inv_freq,
-                               const int R, const float pos,
-                               const float rot_mag, const int lane) {
+                               const int R, const bool interleaved,
+                               const float pos, const float rot_mag,
+                               const int lane) {
   float inv = 1.0f;
-  if (w != nullptr) {
+  if (w != nullptr || unit_norm) {
     float ss = 0.f;
     for (int d = lane; d < D; d += 64) { const float x = act_ld(src + d); ss += x * x; }
     ss = wave_reduce_sum(ss);
     inv = 1.0f / sqrtf(ss / (float)D + eps);
   }
-  for (int d = lane; d < D; d += 64) {
-    float val;
-    if (d < 2 * R) {
-      const int i = d < R ? d : d - R;
-      const float a = act_ld(src + i) * inv * (w ? w[i] : 1.0f);
-      const float b = act_ld(src + i + R) * inv * (w ? w[i + R] : 1.0f);
-      const float ang = pos * inv_freq[i];
-      const float c = cosf(ang) * rot_mag, sn = sinf(ang) * rot_mag;
-      val = d < R ? a * c - b * sn : b * c + a * sn;
-    } else {
-      val = act_ld(src + d) * inv * (w ? w[d] : 1.0f);
-    }
-    act_st(dst + d, val);
+  for (int i = lane; i < R; i += 64) {       // one pair per lane
+    const int da = interleaved ? 2 * i : i;
+    const int db = interleaved ? 2 * i + 1 : i + R;
+    const float a = act_ld(src + da) * inv * (w ? w[da] : 1.0f);
+    const float b = act_ld(src + db) * inv * (w ? w[db] : 1.0f);
+    float sn, c;
+    sincosf(pos * inv_freq[i], &sn, &c);
+    c *= rot_mag;
+    sn *= rot_mag;
+    act_st(dst + da, a * c - b * sn);
+    act_st(dst + db, b * c + a * sn);
   }
+  for (int d = 2 * R + lane; d < D; d += 64)
+    act_st(dst + d, act_ld(src + d) * inv * (w ? w[d] : 1.0f));
 }
 
 template <typename T>
@@ -78,14 +88,15 @@ __global__ void qk_norm_cache_write_kernel(
     const int64_t* __restrict__ slots, const int H, const int G, const int D,
     const int V, const int BS, const int64_t* __restrict__ positions,
     const float* __restrict__ inv_freq, const int R, const float rot_mag,
+    const bool unit_norm, const bool interleaved,
     const T* __restrict__ v_first, const int64_t vf_s0, const int64_t vf_s1,
     const float v_lambda) {
   const int t = blockIdx.x, y = blockIdx.y, lane = threadIdx.x;
   const float pos = R > 0 ? (float)positions[t] : 0.0f;
   if (y < H) {
     norm_rotate_row(q_out + ((int64_t)t * H + y) * D,
-                    q + (int64_t)t * q_s0 + (int64_t)y * q_s1, q_w, eps, D,
-                    inv_freq, R, pos, rot_mag, lane);
+                    q + (int64_t)t * q_s0 + (int64_t)y * q_s1, q_w, unit_norm,
+                    eps, D, inv_freq, R, interleaved, pos, rot_mag, lane);
     return;
   }
   const int64_t slot = slots[t];
@@ -95,8 +106,8 @@ __global__ void qk_norm_cache_write_kernel(
   if (y < H + G) {
     const int g = y - H;
     norm_rotate_row(k_cache + ((blk * G + g) * BS + off) * D,
-                    k + (int64_t)t * k_s0 + (int64_t)g * k_s1, k_w, eps, D,
-                    inv_freq, R, pos, rot_mag, lane);
+                    k + (int64_t)t * k_s0 + (int64_t)g * k_s1, k_w, unit_norm,
+                    eps, D, inv_freq, R, interleaved, pos, rot_mag, lane);
   } else {
     const int g = y - H - G;
     const T* src = v + (int64_t)t * v_s0 + (int64_t)g * v_s1;
@@ -160,7 +171,9 @@ __global__ void window_attention_kernel(
     const float scale, const float softcap, const float* __restrict__ r1,
     const float* __restrict__ r2, const int window, const int H, const int G,
     const int D, const int V, const int BS, const int keep_first,
-    const float* __restrict__ sinks, const int chunk) {
+    const float* __restrict__ sinks, const int chunk,
+    const float* __restrict__ pb, const T* __restrict__ gate,
+    const int64_t gate_s0) {
   extern __shared__ float lds[];
   const int KT = blockDim.x;            // keys per tile
   float* q_s = lds;                     // [D]
@@ -194,6 +207,8 @@ __global__ void window_attention_kernel(
 #pragma unroll
   for (int i = 0; i < MAXV; i++) acc[i] = 0.f;
   float m_run = sinks ? sinks[h] : -INFINITY, l_run = sinks ? 1.0f : 0.f;
+  const float hpb = pb ? pb[h] : 0.0f;
+  if (pb) l_run = 1.0f;                 // unnormalised weights
 
   for (int k0 = 0; k0 < nkeys; k0 += KT) {
     const int nk = min(KT, nkeys - k0);
@@ -209,28 +224,34 @@ __global__ void window_attention_kernel(
       if (softcap > 0.f) s = softcap * tanhf(s / softcap);
       if (r1) s -= hr1 * log1pf(hr2 * (float)(pos - j));
     }
-    // tile max
-    float mx = wave_reduce_max(s);
-    if ((tid & 63) == 0) red[tid >> 6] = mx;
-    __syncthreads();
-    if (tid == 0) {
-      float m = red[0];
-      for (int w = 1; w < (KT >> 6); w++) m = fmaxf(m, red[w]);
-      bcast[0] = m;
+    float corr = 1.0f;
+    if (pb) {
+      p_s[tid] = tid < nk ? sigmoid_f(s + hpb) : 0.f;
+      __syncthreads();
+    } else {
+      // tile max
+      float mx = wave_reduce_max(s);
+      if ((tid & 63) == 0) red[tid >> 6] = mx;
+      __syncthreads();
+      if (tid == 0) {
+        float m = red[0];
+        for (int w = 1; w < (KT >> 6); w++) m = fmaxf(m, red[w]);
+        bcast[0] = m;
+      }
+      __syncthreads();
+      const float m_new = fmaxf(m_run, bcast[0]);
+      const float p = tid < nk ? expf(s - m_new) : 0.f;
+      p_s[tid] = p;
+      float ps = wave_reduce_sum(p);
+      __syncthreads();                  // red[] free again; p_s visible
+      if ((tid & 63) == 0) red[tid >> 6] = ps;
+      __syncthreads();
+      float tile_sum = 0.f;
+      for (int w = 0; w < (KT >> 6); w++) tile_sum += red[w];
+      corr = expf(m_run - m_new);               // 0 on the first tile
+      l_run = l_run * corr + tile_sum;
+      m_run = m_new;
     }
-    __syncthreads();
-    const float m_new = fmaxf(m_run, bcast[0]);
-    const float p = tid < nk ? expf(s - m_new) : 0.f;
-    p_s[tid] = p;
-    float ps = wave_reduce_sum(p);
-    __syncthreads();                    // red[] free again; p_s visible
-    if ((tid & 63) == 0) red[tid >> 6] = ps;
-    __syncthreads();
-    float tile_sum = 0.f;
-    for (int w = 0; w < (KT >> 6); w++) tile_sum += red[w];
-    const float corr = expf(m_run - m_new);     // 0 on the first tile
-    l_run = l_run * corr + tile_sum;
-    m_run = m_new;
 #pragma unroll
     for (int i = 0; i < MAXV; i++) {
       const int j = tid + i * KT;
@@ -242,7 +263,8 @@ __global__ void window_attention_kernel(
       }
     }
   }
-  const float inv = 1.0f / l_run;
+  float inv = 1.0f / l_run;
+  if (gate) inv *= sigmoid_f(act_ld(gate + (int64_t)t * gate_s0 + h));
 #pragma unroll
   for (int i = 0; i < MAXV; i++) {
     const int j = tid + i * KT;
@@ -263,7 +285,7 @@ constexpr int WQ_TILE = 64;
 constexpr int WKV_TILE = 32;
 constexpr int WPAD = 40;
 
-template <int D, int DV>
+template <int D, int DV, bool SIG>
 __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
     short* __restrict__ out,              // [T, H, DV]
     const short* __restrict__ q,          // [T, H, D]
@@ -275,7 +297,8 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
     const float scale, const float softcap, const float* __restrict__ r1,
     const float* __restrict__ r2, const int window, const int H, const int G,
     const int BS, const int keep_first, const float* __restrict__ sinks,
-    const int chunk) {
+    const int chunk, const float* __restrict__ pb,
+    const short* __restrict__ gate, const int64_t gate_s0) {
   constexpr int KK = D / 32;
   constexpr int DT = DV / 16;
   const int tile = blockIdx.x;
@@ -290,6 +313,7 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   const int* bt = block_tables + (int64_t)seq * max_blocks;
   const float hr1 = r1 ? r1[h] : 0.f, hr2 = r1 ? r2[h] : 0.f;
   const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
+  const float hpb = SIG ? pb[h] : 0.f;
 
   const int wave = threadIdx.x >> 6;
   const int lane = threadIdx.x & 63;
@@ -316,7 +340,7 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
 #pragma unroll
   for (int r = 0; r < 4; r++) {
     mrow[r] = sinks ? sinks[h] : -1e30f;
-    lrow[r] = sinks ? 1.0f : 0.f;
+    lrow[r] = sinks || SIG ? 1.0f : 0.f;
   }
 #pragma unroll
   for (int dt = 0; dt < DT; dt++) ofrag[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -385,10 +409,11 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
         if (dist < 0 || kvp >= kv_len || qr >= q_len ||
             (window > 0 && dist >= window && kvp >= keep_first) ||
             (chunk > 0 && kvp < (q_abs / chunk) * chunk)) sv = -1e30f;
-        p[kt][r] = sv;
+        // exp of a masked score's 1e30 is infinite: weight zero
+        p[kt][r] = SIG ? 1.0f / (1.0f + __expf(-(sv + hpb))) : sv;
       }
 #pragma unroll
-    for (int r = 0; r < 4; r++) {
+    for (int r = 0; r < (SIG ? 0 : 4); r++) {
       float mx = fmaxf(p[0][r], p[1][r]);
 #pragma unroll
       for (int off = 1; off < 16; off <<= 1)
@@ -443,7 +468,9 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   for (int r = 0; r < 4; r++) {
     const int qr = q0 + wave * 16 + hi * 4 + r;
     if (qr >= q_len) continue;
-    const float inv = 1.f / fmaxf(lrow[r], 1e-30f);
+    float inv = 1.f / fmaxf(lrow[r], 1e-30f);
+    if (gate)
+      inv *= sigmoid_f(bf16_to_f32(gate[(int64_t)(tok0 + qr) * gate_s0 + h]));
     const int64_t obase = ((int64_t)(tok0 + qr) * H + h) * DV;
 #pragma unroll
     for (int dt = 0; dt < DT; dt++)
@@ -476,7 +503,9 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
     const float scale, const float softcap, const float* __restrict__ r1,
     const float* __restrict__ r2, const int window, const int H, const int G,
     const int D, const int V, const int BS, const int KT,
-    const int keep_first, const float* __restrict__ sinks, const int chunk) {
+    const int keep_first, const float* __restrict__ sinks, const int chunk,
+    const float* __restrict__ pb, const T* __restrict__ gate,
+    const int64_t gate_s0) {
   constexpr int VEC = 16 / (int)sizeof(T);
   extern __shared__ float lds[];
   float* s_s = lds;                            // [RT][KT]
@@ -519,11 +548,12 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
         qreg[r][i][e] = (r < nr && ch < nchunks)
             ? act_ld(q + ((int64_t)t * H + h0 + r) * D + ch * VEC + e) : 0.0f;
     }
-  float hr1[RT], hr2[RT];
+  float hr1[RT], hr2[RT], hpb[RT];
 #pragma unroll
   for (int r = 0; r < RT; r++) {
     hr1[r] = (r1 && r < nr) ? r1[h0 + r] : 0.0f;
     hr2[r] = (r1 && r < nr) ? r2[h0 + r] : 0.0f;
+    hpb[r] = (pb && r < nr) ? pb[h0 + r] : 0.0f;
   }
   // P.V lane roles: LPR lanes cover one value row in 16-byte chunks, so a
   // wave load touches 64 / LPR rows at once
@@ -541,7 +571,8 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
   if (tid < RT) {
     const bool sk = sinks != nullptr && tid < nr;
     m_s[tid] = sk ? sinks[h0 + tid] : -INFINITY;
-    l_s[tid] = sk ? 1.0f : 0.0f;
+    l_s[tid] = sk || pb ? 1.0f : 0.0f;
+    c_s[tid] = 1.0f;
   }
 
   for (int k0 = 0; k0 < nkeys; k0 += KT) {
@@ -593,6 +624,7 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
           float sv = group_reduce_sum<8>(dot) * scale;
           if (softcap > 0.f) sv = softcap * tanhf(sv / softcap);
           if (r1) sv -= hr1[r] * log1pf(hr2[r] * dist);
+          if (pb) sv = sigmoid_f(sv + hpb[r]);
           if (sub == 0 && r < nr && kk < nk) s_s[r * KT + kk] = sv;
         }
         if (sub == 0 && kk < nk) row_s[kk] = rowi[un];
@@ -600,7 +632,8 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
     }
     __syncthreads();
     // ---- softmax statistics of the tile, one head per wave at a time
-    for (int r = wave; r < nr; r += 4) {
+    // (sigmoid weights have none: l and c stay 1)
+    for (int r = pb ? nr : wave; r < nr; r += 4) {
       float mx = -INFINITY;
       for (int kk = lane; kk < nk; kk += 64) mx = fmaxf(mx, s_s[r * KT + kk]);
       mx = wave_reduce_max(mx);
@@ -674,7 +707,9 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
     float a = 0.0f;
 #pragma unroll
     for (int w = 0; w < 4; w++) a += acc_s[(w * RT + r) * 256 + j];
-    act_st(out + ((int64_t)t * H + h0 + r) * V + j, a / l_s[r]);
+    a /= l_s[r];
+    if (gate) a *= sigmoid_f(act_ld(gate + (int64_t)t * gate_s0 + h0 + r));
+    act_st(out + ((int64_t)t * H + h0 + r) * V + j, a);
   }
 }
 
@@ -687,7 +722,8 @@ void launch_decode(int nch, dim3 grid, size_t lds_bytes, hipStream_t stream,
                    float scale, float softcap, const float* r1,
                    const float* r2, int window, int H, int G, int D, int V,
                    int BS, int KT, int keep_first, const float* sinks,
-                   int chunk) {
+                   int chunk, const float* pb, const T* gate,
+                   int64_t gate_s0) {
 #define KAITO_WDEC(NCH_)                                                     \
   if (nch == NCH_) {                                                         \
     hipLaunchKernelGGL((window_attention_decode_kernel<T, RT, NCH_>), grid,  \
@@ -696,7 +732,7 @@ void launch_decode(int nch, dim3 grid, size_t lds_bytes, hipStream_t stream,
         (const T*)v_cache.data_ptr(), block_tables.data_ptr<int>(),          \
         (int)block_tables.size(1), token_seq.data_ptr<int>(),                \
         positions.data_ptr<int64_t>(), scale, softcap, r1, r2, window, H, G, \
-        D, V, BS, KT, keep_first, sinks, chunk);                             \
+        D, V, BS, KT, keep_first, sinks, chunk, pb, gate, gate_s0);          \
     return;                                                                  \
   }
   KAITO_WDEC(1) KAITO_WDEC(2) KAITO_WDEC(4)
@@ -710,6 +746,20 @@ inline bool decode_kernel_fits(int D, int V, int elem) {
   return D % vec == 0 && D / vec <= 32 && V % vec == 0 && V <= 256;
 }
 
+void check_weights_and_gate(const at::Tensor& q, const at::Tensor& sinks,
+                            const at::Tensor& sig_bias,
+                            const at::Tensor& gate) {
+  if (sig_bias.numel() > 0) {
+    KAITO_CHECK_F32(sig_bias);
+    TORCH_CHECK(sig_bias.numel() == q.size(1));
+    TORCH_CHECK(sinks.numel() == 0, "sigmoid weights have no denominator");
+  }
+  if (gate.numel() > 0)
+    TORCH_CHECK(gate.is_cuda() && gate.dim() == 2 && gate.stride(1) == 1 &&
+                gate.dtype() == q.dtype() && gate.size(0) == q.size(0) &&
+                gate.size(1) == q.size(1));
+}
+
 }  // namespace
 
 void qk_norm_cache_write(at::Tensor q_out, at::Tensor q, at::Tensor k,
@@ -717,7 +767,8 @@ void qk_norm_cache_write(at::Tensor q_out, at::Tensor q, at::Tensor k,
                          double eps, at::Tensor k_cache, at::Tensor v_cache,
                          at::Tensor slot_mapping, at::Tensor positions,
                          at::Tensor inv_freq, double rot_mag,
-                         at::Tensor v_first, double v_lambda) {
+                         at::Tensor v_first, double v_lambda, bool unit_norm,
+                         bool interleaved) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && k.dim() == 3 && v.dim() == 3);
   const int T = q.size(0), H = q.size(1), D = q.size(2);
   const int G = k.size(1), V = v.size(2);
@@ -738,6 +789,8 @@ void qk_norm_cache_write(at::Tensor q_out, at::Tensor q, at::Tensor k,
   const bool qn = q_w.numel() > 0, kn = k_w.numel() > 0;
   if (qn) { KAITO_CHECK_F32(q_w); TORCH_CHECK(q_w.numel() == D); }
   if (kn) { KAITO_CHECK_F32(k_w); TORCH_CHECK(k_w.numel() == D); }
+  TORCH_CHECK(!unit_norm || (!qn && !kn && rot_mag == 1.0),
+              "the plain norm takes no weights and no rotation magnitude");
   TORCH_CHECK(slot_mapping.is_cuda() && slot_mapping.dtype() == at::kLong &&
               slot_mapping.is_contiguous() && slot_mapping.size(0) == T);
   const int R = (int)inv_freq.numel();
@@ -765,7 +818,7 @@ void qk_norm_cache_write(at::Tensor q_out, at::Tensor q, at::Tensor k,
         slot_mapping.data_ptr<int64_t>(), H, G, D, V, BS,
         R > 0 ? positions.data_ptr<int64_t>() : nullptr,
         R > 0 ? inv_freq.data_ptr<float>() : nullptr, R, (float)rot_mag,
-        blend ? (const act_t*)v_first.data_ptr() : nullptr,
+        unit_norm, interleaved, blend ? (const act_t*)v_first.data_ptr() : nullptr,
         blend ? v_first.stride(0) : 0, blend ? v_first.stride(1) : 0,
         (float)v_lambda);
   });
@@ -776,7 +829,8 @@ void window_attention(at::Tensor out, at::Tensor q, at::Tensor k_cache,
                       at::Tensor token_seq, at::Tensor positions,
                       double scale, double softcap, at::Tensor r1,
                       at::Tensor r2, int64_t window, int64_t keep_first,
-                      at::Tensor sinks, int64_t chunk) {
+                      at::Tensor sinks, int64_t chunk, at::Tensor sig_bias,
+                      at::Tensor gate) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() &&
               is_act_dtype(q));
   TORCH_CHECK(keep_first >= 0 && keep_first < (1 << 30));
@@ -790,6 +844,10 @@ void window_attention(at::Tensor out, at::Tensor q, at::Tensor k_cache,
     KAITO_CHECK_F32(sinks);
     TORCH_CHECK(sinks.numel() == q.size(1));
   }
+  check_weights_and_gate(q, sinks, sig_bias, gate);
+  const float* pb = sig_bias.numel() > 0 ? sig_bias.data_ptr<float>()
+                                         : nullptr;
+  const bool gated = gate.numel() > 0;
   const int T = q.size(0), H = q.size(1), D = q.size(2);
   TORCH_CHECK(k_cache.is_contiguous() && v_cache.is_contiguous() &&
               k_cache.dim() == 4 && v_cache.dim() == 4 &&
@@ -830,26 +888,28 @@ void window_attention(at::Tensor out, at::Tensor q, at::Tensor k_cache,
     const float* p2 = bias ? r2.data_ptr<float>() : nullptr;
     const float* ps = has_sinks ? sinks.data_ptr<float>() : nullptr;
     KAITO_DISPATCH_ACT(q, {
+      const act_t* pg = gated ? (const act_t*)gate.data_ptr() : nullptr;
+      const int64_t gs0 = gated ? gate.stride(0) : 0;
       if (rt == 8)
         launch_decode<act_t, 8>(nch, grid, lds_bytes, stream0, out, q,
             k_cache, v_cache, block_tables, token_seq, positions,
             (float)scale, (float)softcap, p1, p2, (int)window, H, G, D, V,
-            BS, KT, kf, ps, (int)chunk);
+            BS, KT, kf, ps, (int)chunk, pb, pg, gs0);
       else if (rt == 4)
         launch_decode<act_t, 4>(nch, grid, lds_bytes, stream0, out, q,
             k_cache, v_cache, block_tables, token_seq, positions,
             (float)scale, (float)softcap, p1, p2, (int)window, H, G, D, V,
-            BS, KT, kf, ps, (int)chunk);
+            BS, KT, kf, ps, (int)chunk, pb, pg, gs0);
       else if (rt == 2)
         launch_decode<act_t, 2>(nch, grid, lds_bytes, stream0, out, q,
             k_cache, v_cache, block_tables, token_seq, positions,
             (float)scale, (float)softcap, p1, p2, (int)window, H, G, D, V,
-            BS, KT, kf, ps, (int)chunk);
+            BS, KT, kf, ps, (int)chunk, pb, pg, gs0);
       else
         launch_decode<act_t, 1>(nch, grid, lds_bytes, stream0, out, q,
             k_cache, v_cache, block_tables, token_seq, positions,
             (float)scale, (float)softcap, p1, p2, (int)window, H, G, D, V,
-            BS, KT, kf, ps, (int)chunk);
+            BS, KT, kf, ps, (int)chunk, pb, pg, gs0);
     });
     return;
   }
@@ -871,7 +931,9 @@ void window_attention(at::Tensor out, at::Tensor q, at::Tensor k_cache,
         positions.data_ptr<int64_t>(), (float)scale, (float)softcap,
         bias ? r1.data_ptr<float>() : nullptr,
         bias ? r2.data_ptr<float>() : nullptr, (int)window, H, G, D, V, BS,
-        kf, has_sinks ? sinks.data_ptr<float>() : nullptr, (int)chunk);
+        kf, has_sinks ? sinks.data_ptr<float>() : nullptr, (int)chunk, pb,
+        gated ? (const act_t*)gate.data_ptr() : nullptr,
+        gated ? gate.stride(0) : 0);
   });
 }
 
@@ -885,7 +947,8 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
                             at::Tensor cu_seqlens, at::Tensor seq_starts,
                             double scale, double softcap, at::Tensor r1,
                             at::Tensor r2, int64_t window, int64_t keep_first,
-                            at::Tensor sinks, int64_t chunk) {
+                            at::Tensor sinks, int64_t chunk,
+                            at::Tensor sig_bias, at::Tensor gate) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() &&
               q.dtype() == at::kBFloat16);
   TORCH_CHECK(keep_first >= 0 && keep_first < (1 << 30));
@@ -897,6 +960,10 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
     KAITO_CHECK_F32(sinks);
     TORCH_CHECK(sinks.numel() == q.size(1));
   }
+  check_weights_and_gate(q, sinks, sig_bias, gate);
+  const float* pb = sig_bias.numel() > 0 ? sig_bias.data_ptr<float>()
+                                         : nullptr;
+  const bool gated = gate.numel() > 0;
   const int T = q.size(0), H = q.size(1), D = q.size(2);
   TORCH_CHECK(k_cache.is_contiguous() && v_cache.is_contiguous() &&
               k_cache.dim() == 4 && v_cache.dim() == 4 &&
@@ -922,9 +989,8 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
   const int ntiles = tile_seq.size(0);
   if (ntiles == 0 || T == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
-#define KAITO_WIN_CASE(D_, DV_)                                              \
-  if (D == D_ && V == DV_) {                                                 \
-    hipLaunchKernelGGL((window_attention_mfma_kernel<D_, DV_>),              \
+#define KAITO_WIN_LAUNCH(D_, DV_, SIG_)                                      \
+    hipLaunchKernelGGL((window_attention_mfma_kernel<D_, DV_, SIG_>),        \
         dim3(ntiles, H), dim3(256), 0, stream, (short*)out.data_ptr(),       \
         (const short*)q.data_ptr(), (const short*)k_cache.data_ptr(),        \
         (const short*)v_cache.data_ptr(), tile_seq.data_ptr<int>(),          \
@@ -933,7 +999,13 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
         (int)block_tables.size(1), (float)scale, (float)softcap,             \
         bias ? r1.data_ptr<float>() : nullptr,                               \
         bias ? r2.data_ptr<float>() : nullptr, (int)window, H, G, BS, kf,    \
-        has_sinks ? sinks.data_ptr<float>() : nullptr, (int)chunk);          \
+        has_sinks ? sinks.data_ptr<float>() : nullptr, (int)chunk, pb,       \
+        gated ? (const short*)gate.data_ptr() : nullptr,                     \
+        gated ? gate.stride(0) : 0)
+#define KAITO_WIN_CASE(D_, DV_)                                              \
+  if (D == D_ && V == DV_) {                                                 \
+    if (pb) KAITO_WIN_LAUNCH(D_, DV_, true);                                 \
+    else KAITO_WIN_LAUNCH(D_, DV_, false);                                   \
     return;                                                                  \
   }
   KAITO_WIN_CASE(64, 64) KAITO_WIN_CASE(64, 128) KAITO_WIN_CASE(128, 64)
@@ -941,6 +1013,7 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
   KAITO_WIN_CASE(256, 256) KAITO_WIN_CASE(64, 256) KAITO_WIN_CASE(256, 64)
   KAITO_WIN_CASE(64, 32) KAITO_WIN_CASE(128, 32) KAITO_WIN_CASE(256, 32)
 #undef KAITO_WIN_CASE
+#undef KAITO_WIN_LAUNCH
   TORCH_CHECK(false, "window_attention_tiles: key sizes {64, 128, 256} and "
               "value sizes {32, 64, 128, 256}, got ", D, "/", V);
 }
@@ -948,9 +1021,9 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
 }  // namespace kaito
 
 TORCH_LIBRARY_FRAGMENT(kaito, m) {
-  m.def("window_attention_tiles(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tile_seq, Tensor tile_qbase, Tensor cu_seqlens, Tensor seq_starts, float scale, float softcap, Tensor r1, Tensor r2, int window, int keep_first, Tensor sinks, int chunk) -> ()");
-  m.def("qk_norm_cache_write(Tensor(a!) q_out, Tensor q, Tensor k, Tensor v, Tensor q_w, Tensor k_w, float eps, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slot_mapping, Tensor positions, Tensor inv_freq, float rot_mag, Tensor v_first, float v_lambda) -> ()");
-  m.def("window_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor token_seq, Tensor positions, float scale, float softcap, Tensor r1, Tensor r2, int window, int keep_first, Tensor sinks, int chunk) -> ()");
+  m.def("window_attention_tiles(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tile_seq, Tensor tile_qbase, Tensor cu_seqlens, Tensor seq_starts, float scale, float softcap, Tensor r1, Tensor r2, int window, int keep_first, Tensor sinks, int chunk, Tensor sig_bias, Tensor gate) -> ()");
+  m.def("qk_norm_cache_write(Tensor(a!) q_out, Tensor q, Tensor k, Tensor v, Tensor q_w, Tensor k_w, float eps, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slot_mapping, Tensor positions, Tensor inv_freq, float rot_mag, Tensor v_first, float v_lambda, bool unit_norm, bool interleaved) -> ()");
+  m.def("window_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor token_seq, Tensor positions, float scale, float softcap, Tensor r1, Tensor r2, int window, int keep_first, Tensor sinks, int chunk, Tensor sig_bias, Tensor gate) -> ()");
 }
 TORCH_LIBRARY_IMPL(kaito, CUDA, m) {
   m.impl("qk_norm_cache_write", &kaito::qk_norm_cache_write);

@@ -348,11 +348,14 @@ def rglru_scan(u, gates, y, decay_rate, state, cu_seqlens, state_slots,
 def qk_norm_cache_write(q, k, v, q_w, k_w, eps: float, k_cache, v_cache,
                         slot_mapping, positions=None, inv_freq=None,
                         rot_mag: float = 1.0, v_first=None,
-                        v_lambda: float = 0.0):
+                        v_lambda: float = 0.0, unit_norm: bool = False,
+                        interleaved: bool = False):
     """Per-head RMS norm of q [T, H, D] and k [T, G, D] (weights [D], or
     None for no norm), optional rotation of the first 2*len(inv_freq)
-    dims of every head (dim i paired with i + len(inv_freq); angle =
-    position * inv_freq[i]; cos and sin times rot_mag), optional blend
+    dims of every head (dim i paired with i + len(inv_freq), or with
+    `interleaved` dim 2i with 2i + 1; angle =
+    position * inv_freq[i]; cos and sin times rot_mag), with `unit_norm`
+    a plain RMS norm per head after the rotation, optional blend
     v <- (1 - v_lambda) v + v_lambda v_first, then scatter k and v
     [T, G, V] into the paged caches [blocks, G, block_size, D|V].
     Returns the normed (rotated) q."""
@@ -370,11 +373,20 @@ def qk_norm_cache_write(q, k, v, q_w, k_w, eps: float, k_cache, v_cache,
         ang = positions.float()[:, None] * inv_freq.float()[None, :]
         c = (torch.cos(ang) * rot_mag)[:, None, :]
         s = (torch.sin(ang) * rot_mag)[:, None, :]
+        if interleaved:
+            a, b = tf[..., 0:2 * half:2], tf[..., 1:2 * half:2]
+            pairs = torch.stack([a * c - b * s, b * c + a * s], -1).flatten(-2)
+            return torch.cat([pairs, tf[..., 2 * half:]], -1)
         a, b = tf[..., :half], tf[..., half:2 * half]
         return torch.cat([a * c - b * s, b * c + a * s, tf[..., 2 * half:]],
                          -1)
-    qn = rot(norm(q, q_w)).to(q.dtype)
-    kn = rot(norm(k, k_w)).to(k.dtype)
+
+    def plain(tf):
+        if unit_norm:
+            tf = tf * torch.rsqrt(tf.pow(2).mean(-1, keepdim=True) + eps)
+        return tf
+    qn = plain(rot(norm(q, q_w))).to(q.dtype)
+    kn = plain(rot(norm(k, k_w))).to(k.dtype)
     if v_first is not None:
         v = ((1.0 - v_lambda) * v.float() + v_lambda * v_first.float()) \
             .to(v.dtype)
@@ -389,7 +401,8 @@ def qk_norm_cache_write(q, k, v, q_w, k_w, eps: float, k_cache, v_cache,
 
 def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
                      scale: float, softcap: float, r1, r2, window: int,
-                     keep_first: int = 0, sinks=None, chunk: int = 0):
+                     keep_first: int = 0, sinks=None, chunk: int = 0,
+                     sigmoid_bias=None, gate=None):
     """Causal sliding-window attention of query rows over the paged cache.
     Row t belongs to chunk token_seq[t] (its block table row) at sequence
     position positions[t] and sees keys j <= pos with pos - j < window or
@@ -397,7 +410,8 @@ def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
     cap(q.k * scale) - r1 * ln(1 + r2 * (pos - j)). With `sinks` [H] the
     softmax denominator also holds exp(sink_h). With `chunk` > 0 the mask
     is chunked instead: keys j <= pos in pos's block of `chunk` positions
-    counted from 0."""
+    counted from 0. With `sigmoid_bias` [H] a key's weight is sigmoid(score
+    + bias), not normalised. `gate` [T, H]: outputs times sigmoid(gate)."""
     T, H, D = q.shape
     G, bs, V = k_cache.size(1), k_cache.size(2), v_cache.size(3)
     rep = H // G
@@ -424,12 +438,16 @@ def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
             dist = (p - js).float()
             s = s - r1.float()[:, None] * torch.log1p(
                 r2.float()[:, None] * dist[None, :])
-        if sinks is not None:
+        if sigmoid_bias is not None:
+            w = torch.sigmoid(s + sigmoid_bias.float()[:, None])
+        elif sinks is not None:
             s = torch.cat([s, sinks.float()[:, None]], 1)
             w = torch.softmax(s, -1)[:, :-1]
         else:
             w = torch.softmax(s, -1)
         out[t] = torch.einsum("hn,nhv->hv", w, vv)
+        if gate is not None:
+            out[t] *= torch.sigmoid(gate[t].float())[:, None]
     return out.to(q.dtype)
 
 
@@ -565,6 +583,13 @@ def gelu_glu(gu):
     F_ = gu.size(-1) // 2
     g = torch.nn.functional.gelu(gu[..., :F_].float(), approximate="tanh")
     return (g * gu[..., F_:].float()).to(gu.dtype)
+
+
+def relu_glu(gu):
+    """gu [T, 2F] = [gate | up] -> relu(gate) * up."""
+    F_ = gu.size(-1) // 2
+    return (torch.relu(gu[..., :F_].float()) * gu[..., F_:].float()) \
+        .to(gu.dtype)
 
 
 def relu2(x):
@@ -755,3 +780,65 @@ def hgrn2_scan(q, v, f_pre, lower, norm_w, state, cu_seqlens, state_slots,
     out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + norm_eps) \
         * norm_w.float()
     return out.reshape(T, H * V).to(q.dtype)
+
+
+def moe_route(logits, correction, top: int, n_real: int, groups: int,
+              keep: int, renorm: bool, scale: float):
+    """Softmax scores; choice by score + correction among the `keep` groups
+    with the largest choice; weights are the scores. Returns (indices
+    [T, top] int32, weights [T, top] f32, weight [T] on outputs >=
+    n_real)."""
+    T, N = logits.shape
+    s = torch.softmax(logits.float(), -1)
+    choice = s + correction.float()
+    if groups > 1:
+        best = choice.view(T, groups, -1).amax(-1).topk(keep, -1)[1]
+        ok = torch.zeros(T, groups, dtype=torch.bool, device=logits.device)
+        ok.scatter_(1, best, True)
+        choice = choice.masked_fill(
+            ~ok.repeat_interleave(N // groups, 1), float("-inf"))
+    topi = choice.topk(top, -1)[1]
+    w = s.gather(1, topi)
+    if renorm:
+        w = w / (w.sum(-1, keepdim=True) + 1e-20)
+    w = w * scale
+    return topi.to(torch.int32), w, (w * (topi >= n_real)).sum(-1)
+
+
+def moe_sort(topi, topw, n: int):
+    """Stable sort of the (token, expert) pairs by expert: (token, weight,
+    exclusive offsets [n + 1])."""
+    flat = topi.reshape(-1).long()
+    order = torch.argsort(flat, stable=True)
+    offsets = torch.zeros(n + 1, dtype=torch.int32, device=topi.device)
+    offsets[1:] = torch.cumsum(torch.bincount(flat, minlength=n), 0)
+    return ((order // topi.size(1)).to(torch.int32),
+            topw.reshape(-1)[order].float(), offsets)
+
+
+def _stream_norm(u, w, eps: float, out_dtype):
+    return (u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eps)
+            * w.float()).to(out_dtype)
+
+
+def stream_embed(ids, table, g, w_in, w, eps: float):
+    """S = len(w_in) equal streams [T, S, H] f32 of rms(table[ids])*g, and
+    rms(sum_s w_in[s] x_s)*w."""
+    x = _stream_norm(table[ids].float(), g, eps, torch.float32)
+    x = x[:, None, :].repeat(1, w_in.numel(), 1)
+    u = (x * w_in.float()[None, :, None]).sum(1)
+    return x, _stream_norm(u, w, eps, table.dtype)
+
+
+def stream_mix_norm(x, y, mix, w_out, w_in, w, eps: float, out_dtype,
+                    write_x: bool = True):
+    """x [T, S, H] f32: x_t <- sum_s mix[s, t] x_s + w_out[t]*y in place;
+    returns u = sum_s w_in[s] x_s of the new streams, normed with w unless
+    w is None."""
+    new = torch.einsum("nsh,st->nth", x, mix.float()) \
+        + w_out.float()[None, :, None] * y.float()[:, None, :]
+    if write_x:
+        x.copy_(new)
+    u = (new * w_in.float()[None, :, None]).sum(1)
+    return u.to(out_dtype) if w is None else _stream_norm(u, w, eps,
+                                                          out_dtype)

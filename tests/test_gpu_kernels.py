@@ -692,8 +692,9 @@ def test_moe_fused_grouped_gemms(T, H, IE, E, K):
         for p in m.parameters():
             p.normal_(0, 0.05)
     x = _bf16(T, H, scale=0.5)
-    sorted_tok, gates, offsets = m._route(x)
-    out_fused = m._forward_fused(x, sorted_tok, gates, offsets)
+    sorted_tok, gates, offsets, _ = m._route(x)
+    out_fused = torch.zeros(T, H, dtype=torch.float32, device=DEV)
+    m._forward_fused(x, sorted_tok, gates, offsets, out_fused)
     # fp32 oracle on the same routing
     off = offsets.tolist()
     expect = torch.zeros(T, H, dtype=torch.float32, device=DEV)

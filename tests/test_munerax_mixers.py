@@ -421,7 +421,8 @@ def test_group_limited_routing_choices():
         W[f"r.e{e}.down"] = np.zeros((6, 4))
     mlp = M.moe(6, 2, 4, scale=1.5, groups=(3, 1))
     m = moe_module("cpu", torch.float32, 6, mlp, W, "r.")
-    tok, gates, offsets = m._route(torch.tensor(z, dtype=torch.float32)[None])
+    tok, gates, offsets, _ = m._route(
+        torch.tensor(z, dtype=torch.float32)[None])
     counts = (offsets[1:] - offsets[:-1]).tolist()
     assert counts == [0, 0, 1, 1, 0, 0]
     assert torch.allclose(gates.double(), torch.tensor(
@@ -480,13 +481,13 @@ def test_element_wise_gates(mode):
 
 @pytest.mark.parametrize("mode", MODES)
 def test_dense_feed_forward(mode):
-    from kaito_amd.models.hybrid_config import GeluGLUSpec
-    from kaito_amd.models.mixers import GeluGLU
+    from kaito_amd.models.hybrid_config import GLUSpec
+    from kaito_amd.models.mixers import GatedFF
     dev, dt = mode
     cfg = M.make_config([M.latent_layer(1, 4, 2, 4, 4, mlp=M.dense(36))],
                         width=20, vocab=8, bigram=None)
     W = M.random_weights(cfg, seed=8)
-    m = GeluGLU(20, GeluGLUSpec(36), dt).to(dev)
+    m = GatedFF(20, GLUSpec(36), dt).to(dev)
     with torch.no_grad():
         m.gate_up.copy_(torch.cat([torch.tensor(W["l0.mlp.gate"]),
                                    torch.tensor(W["l0.mlp.up"])], 0).to(dt))
