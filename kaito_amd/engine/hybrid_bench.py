@@ -1,8 +1,8 @@
 """Prefill and decode throughput of the hybrid stacks (Gurapel, Pokulorn,
-Munerax, Lokedra) beside each other and beside the engine's closest homogeneous
+Munerax, Lokedra, Vemenex) beside each other and beside the engine's closest homogeneous
 model at equal size: a sliding-window GQA transformer with the same MoE
-feed-forward (the gpt-oss class without sinks) for the recurrent hybrids,
-the latent-attention MoE transformer (deepseek class) for Munerax. Random
+feed-forward (the gpt-oss class without sinks) for the recurrent hybrids
+and Vemenex, the latent-attention MoE transformer (deepseek class) for Munerax. Random
 weights, synthetic tokens; all models run through the same LLMEngine
 (scheduler, paged cache, hipGraph decode).
 
@@ -178,6 +178,35 @@ def lokedra_config(name: str, z: dict, max_pos: int):
         "vocab": z["vocab"], "width": z["width"]}, name=f"lokedra-{name}")
 
 
+def vemenex_config(name: str, z: dict, max_pos: int):
+    """The hyper-connected stack at the sizes of `z`: sigmoid-weight and
+    unit-sink attention in turn, four residual streams, routed experts of
+    the same count and width (two groups of which one is eligible, two
+    identity outputs beside the experts) in every layer but a dense
+    first."""
+    from ..models.hybrid_config import vemenex_model_config
+    moe = {"kind": "moe", "expert": {"ff": z["ff"], "limit": 7.0},
+           "router": {"experts": z["experts"], "top": z["top"],
+                      "identity": 2, "groups": {"count": 2, "keep": 1}}}
+    dense = {"kind": "dense", "ff": z["ff"] * z["top"]}
+
+    def layer(i):
+        rot = {"base": 10000.0, "dims": z["dim"]}
+        if i % 2 == 0:
+            rot["scaling"] = {"factor": 4.0}
+        return {"type": "attention" if i % 2 == 0 else "attention_2",
+                "mlp": dense if i == 0 else moe, "mixer": {
+                    "heads": z["heads"], "kv_heads": z["kv_heads"],
+                    "dim": z["dim"], "vdim": z["dim"], "rot": rot,
+                    "mask": {"size": z["window"]},
+                    "scale": z["dim"] ** -0.5}}
+    return vemenex_model_config({
+        "architecture": "Vemenex", "streams": 4, "residual_mult": 0.5,
+        "layers": [layer(i) for i in range(z["layers"])],
+        "max_positions": max_pos, "norm": {"eps": 1e-5},
+        "vocab": z["vocab"], "width": z["width"]}, name=f"vemenex-{name}")
+
+
 def latent_transformer_config(name: str, z: dict, max_pos: int):
     """The engine's latent-attention MoE transformer (deepseek class) with
     the same head layout, latent rank, experts, groups and shared
@@ -257,6 +286,7 @@ def run(sizes: List[str], batch: int, prompt: int, out_tokens: int,
                     "swa-moe": transformer_config,
                     "munerax": munerax_config,
                     "lokedra": lokedra_config,
+                    "vemenex": vemenex_config,
                     "mla-moe": latent_transformer_config}[kind](
                         name, z, max_pos)
             pre, dec = _measure(mcfg, batch, prompt, out_tokens, eager)
