@@ -150,6 +150,63 @@ __global__ void stream_mix_norm_any_kernel(
   }
 }
 
+template <int NV, typename T>
+__global__ __launch_bounds__(512) void stream_embed_wide_kernel(
+    float* __restrict__ x, T* __restrict__ h_out,
+    const int64_t* __restrict__ ids, const T* __restrict__ table,
+    const float* __restrict__ g, const int g_step,
+    const float* __restrict__ w_in, const float* __restrict__ w,
+    const int w_step, const int vocab, const int S, const int H,
+    const float eps) {
+  __shared__ float red[16];
+  const int64_t row = blockIdx.x;
+  const int64_t id = ids[row];
+  const bool ok = id >= 0 && id < vocab;    // other ids: a row of zeros
+  const T* src = table + (ok ? id : 0) * H;
+  float* xr = x + row * S * H;
+  const int nvec = H / 4;
+  float cin = 0.f;
+  for (int s = 0; s < S; s++) cin += w_in[s];
+  float4_t v[NV];
+  float ss = 0.f;
+#pragma unroll
+  for (int n = 0; n < NV; n++) {
+    const int i = threadIdx.x + n * blockDim.x;
+    v[n] = i < nvec && ok ? act_ld4(src + i * 4)
+                          : float4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int e = 0; e < 4; e++) ss += v[n][e] * v[n][e];
+  }
+  ss = block_reduce_sum(ss, red);
+  __syncthreads();                          // red[] is used again below
+  const float inv = 1.0f / sqrtf(ss / (float)H + eps);
+  float su = 0.f;
+#pragma unroll
+  for (int n = 0; n < NV; n++) {
+    const int i = threadIdx.x + n * blockDim.x;
+    if (i >= nvec) continue;
+#pragma unroll
+    for (int e = 0; e < 4; e++) {
+      v[n][e] *= inv * g[(i * 4 + e) * g_step];
+      const float u = cin * v[n][e];
+      su += u * u;
+    }
+    for (int s = 0; s < S; s++) act_st4(xr + (int64_t)s * H + i * 4, v[n]);
+  }
+  su = block_reduce_sum(su, red);
+  const float inv_u = 1.0f / sqrtf(su / (float)H + eps);
+#pragma unroll
+  for (int n = 0; n < NV; n++) {
+    const int i = threadIdx.x + n * blockDim.x;
+    if (i >= nvec) continue;
+    float4_t o;
+#pragma unroll
+    for (int e = 0; e < 4; e++)
+      o[e] = cin * v[n][e] * inv_u * w[(i * 4 + e) * w_step];
+    act_st4(h_out + row * H + i * 4, o);
+  }
+}
+
 template <typename T>
 __global__ void stream_embed_kernel(
     float* __restrict__ x, T* __restrict__ h_out,
@@ -285,12 +342,25 @@ void stream_embed(at::Tensor x, at::Tensor h_out, at::Tensor ids,
   if (T == 0 || H == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
   KAITO_DISPATCH_ACT(table, {
-    hipLaunchKernelGGL((stream_embed_kernel<act_t>), dim3(T),
-        dim3(row_threads(H)), 0, stream, x.data_ptr<float>(),
-        (act_t*)h_out.data_ptr(), ids.data_ptr<int64_t>(),
-        (const act_t*)table.data_ptr(), g.data_ptr<float>(),
-        weight_step(g, H), w_in.data_ptr<float>(), w.data_ptr<float>(),
-        weight_step(w, H), (int)table.size(0), S, H, (float)eps);
+    auto launch = [&](auto kernel, int threads) {
+      hipLaunchKernelGGL(kernel, dim3(T), dim3(threads), 0, stream,
+          x.data_ptr<float>(), (act_t*)h_out.data_ptr(),
+          ids.data_ptr<int64_t>(), (const act_t*)table.data_ptr(),
+          g.data_ptr<float>(), weight_step(g, H), w_in.data_ptr<float>(),
+          w.data_ptr<float>(), weight_step(w, H), (int)table.size(0), S, H,
+          (float)eps);
+    };
+    if (H % 4 == 0 && H <= 8192 &&
+        (uintptr_t)table.data_ptr() % (4 * sizeof(act_t)) == 0 &&
+        (uintptr_t)h_out.data_ptr() % (4 * sizeof(act_t)) == 0) {
+      const int threads = std::min(512, (H / 4 + 63) / 64 * 64);
+      if (H / 4 <= threads)
+        launch(stream_embed_wide_kernel<1, act_t>, threads);
+      else
+        launch(stream_embed_wide_kernel<4, act_t>, threads);
+    } else {
+      launch(stream_embed_kernel<act_t>, row_threads(H));
+    }
   });
 }
 

@@ -123,6 +123,130 @@ __global__ void qk_norm_cache_write_kernel(
   }
 }
 
+// One workgroup per token (per pass over a token's rows in small steps).
+// The rotation's cos and sin do not depend on the head: they are computed
+// once into LDS, while the first rows are on their way. LPR lanes hold a row in 16-byte
+// chunks, so a wave covers 64 / LPR rows; the statistic is a shuffle sum over
+// them, and for halves pairing a chunk's partner is R / VEC lanes away.
+constexpr int QKN_MAX_R = 256;
+
+template <typename T>
+__global__ __launch_bounds__(256) void qk_norm_cache_write_vec_kernel(
+    T* __restrict__ q_out,                                   // [T, H, D]
+    const T* __restrict__ q, const int64_t q_s0, const int64_t q_s1,
+    const T* __restrict__ k, const int64_t k_s0, const int64_t k_s1,
+    const T* __restrict__ v, const int64_t v_s0, const int64_t v_s1,
+    const float* __restrict__ q_w, const float* __restrict__ k_w,
+    const float eps, T* __restrict__ k_cache, T* __restrict__ v_cache,
+    const int64_t* __restrict__ slots, const int H, const int G, const int D,
+    const int V, const int BS, const int64_t* __restrict__ positions,
+    const float* __restrict__ inv_freq, const int R, const float rot_mag,
+    const bool unit_norm, const bool interleaved,
+    const T* __restrict__ v_first, const int64_t vf_s0, const int64_t vf_s1,
+    const float v_lambda, const int LPR) {
+  constexpr int VEC = 16 / (int)sizeof(T);
+  __shared__ float cs[QKN_MAX_R], sn[QKN_MAX_R];
+  const int64_t t = blockIdx.x;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int sub = tid % LPR, grp = tid / LPR, rpp = 256 / LPR;
+  const int rows = H + 2 * G, col = sub * VEC, RL = R / VEC;
+  const int64_t slot = slots[t];
+  auto fetch = [&](const int y) {
+    const bool is_v = y >= H + G;
+    float4_t raw{0.f, 0.f, 0.f, 0.f};
+    if (y < rows && col < (is_v ? V : D)) {
+      const int g = y - H - (is_v ? G : 0);
+      raw = *reinterpret_cast<const float4_t*>(
+          (y < H ? q + t * q_s0 + (int64_t)y * q_s1
+                 : (is_v ? v + t * v_s0 + (int64_t)g * v_s1
+                         : k + t * k_s0 + (int64_t)g * k_s1)) + col);
+    }
+    return raw;
+  };
+  int y = blockIdx.y * rpp + grp;
+  float4_t nxt = fetch(y);
+  if (R > 0) {
+    const float pos = (float)positions[t];
+    for (int i = tid; i < R; i += 256) {
+      float s, c;
+      sincosf(pos * inv_freq[i], &s, &c);
+      cs[i] = c * rot_mag;
+      sn[i] = s * rot_mag;
+    }
+  }
+  __syncthreads();
+  const int64_t blk = slot < 0 ? 0 : slot / BS;
+  const int off = slot < 0 ? 0 : (int)(slot % BS);
+  // same trips in all lanes
+  for (int y0 = blockIdx.y * rpp; y0 < rows; y0 += gridDim.y * rpp) {
+    y = y0 + grp;
+    const bool is_q = y < H, is_v = y >= H + G;
+    const int g = y - H - (is_v ? G : 0);
+    const bool in = y < rows && col < (is_v ? V : D);
+    alignas(16) T raw[VEC];
+    *reinterpret_cast<float4_t*>(raw) = nxt;
+    nxt = fetch(y + gridDim.y * rpp);
+    float val[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; e++) val[e] = act_ld(raw + e);
+    const float* w = is_v ? nullptr : (is_q ? q_w : k_w);
+    if (q_w != nullptr || k_w != nullptr || unit_norm) {
+      float ss = 0.f;
+#pragma unroll
+      for (int e = 0; e < VEC; e++) ss += val[e] * val[e];
+      for (int o = 1; o < LPR; o <<= 1) ss += __shfl_xor(ss, o, 64);
+      const float inv = 1.0f / sqrtf(ss / (float)D + eps);
+      if (w != nullptr || (unit_norm && !is_v)) {
+#pragma unroll
+        for (int e = 0; e < VEC; e++)
+          val[e] *= inv * (w && in ? w[col + e] : 1.0f);
+      }
+    }
+    if (R > 0 && interleaved) {
+      if (!is_v) {
+#pragma unroll
+        for (int e = 0; e < VEC; e += 2) {
+          if (col + e < 2 * R) {
+            const int i = (col + e) >> 1;
+            const float a = val[e], b = val[e + 1];
+            val[e] = a * cs[i] - b * sn[i];
+            val[e + 1] = b * cs[i] + a * sn[i];
+          }
+        }
+      }
+    } else if (R > 0) {
+      const bool first = sub < RL, rot = sub < 2 * RL;
+      const int from = (lane & ~(LPR - 1)) +
+          (first ? sub + RL : (rot ? sub - RL : sub));
+#pragma unroll
+      for (int e = 0; e < VEC; e++) {
+        const float other = __shfl(val[e], from, 64);
+        if (rot && !is_v) {
+          const int i = (first ? sub : sub - RL) * VEC + e;
+          val[e] = first ? val[e] * cs[i] - other * sn[i]
+                         : val[e] * cs[i] + other * sn[i];
+        }
+      }
+    }
+    if (!in || (!is_q && slot < 0)) continue;
+    if (is_v && v_first != nullptr) {
+      *reinterpret_cast<float4_t*>(raw) =
+          *reinterpret_cast<const float4_t*>(
+              v_first + t * vf_s0 + (int64_t)g * vf_s1 + col);
+#pragma unroll
+      for (int e = 0; e < VEC; e++)
+        val[e] = (1.0f - v_lambda) * val[e] + v_lambda * act_ld(raw + e);
+    }
+    T* dst = is_q ? q_out + (t * H + y) * D
+        : (is_v ? v_cache + ((blk * G + g) * BS + off) * V
+                : k_cache + ((blk * G + g) * BS + off) * D);
+#pragma unroll
+    for (int e = 0; e < VEC; e++) act_st(raw + e, val[e]);
+    *reinterpret_cast<float4_t*>(dst + col) =
+        *reinterpret_cast<const float4_t*>(raw);
+  }
+}
+
 // ---- attention ------------------------------------------------------------
 template <typename T>
 KAITO_DEV float dot_row(const float* __restrict__ q, const T* __restrict__ k,
@@ -806,7 +930,41 @@ void qk_norm_cache_write(at::Tensor q_out, at::Tensor q, at::Tensor k,
                 v_first.stride(2) == 1 && v_first.dtype() == v.dtype());
   if (T == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
+  // 16-byte rows: every row start, page row and rotated chunk aligned
+  const int vec = 16 / (int)q.element_size();
+  auto rows16 = [&](const at::Tensor& x) {
+    return (uintptr_t)x.data_ptr() % 16 == 0 && x.stride(0) % vec == 0 &&
+        x.stride(1) % vec == 0;
+  };
+  const int chunks = std::max(D, V) / vec;
+  int lpr = 1;
+  while (lpr < chunks) lpr <<= 1;
+  const bool wide = D % vec == 0 && V % vec == 0 && lpr <= 64 &&
+      R <= QKN_MAX_R && (interleaved || R % vec == 0) && qn == kn &&
+      rows16(q) && rows16(k) && rows16(v) && (!blend || rows16(v_first)) &&
+      (uintptr_t)q_out.data_ptr() % 16 == 0 &&
+      (uintptr_t)k_cache.data_ptr() % 16 == 0 &&
+      (uintptr_t)v_cache.data_ptr() % 16 == 0;
   KAITO_DISPATCH_ACT(q, {
+    if (wide) {
+      hipLaunchKernelGGL((qk_norm_cache_write_vec_kernel<act_t>),
+          dim3(T, T < 512 ? (H + 2 * G + 256 / lpr - 1) / (256 / lpr) : 1),
+          dim3(256), 0, stream, (act_t*)q_out.data_ptr(),
+          (const act_t*)q.data_ptr(), q.stride(0), q.stride(1),
+          (const act_t*)k.data_ptr(), k.stride(0), k.stride(1),
+          (const act_t*)v.data_ptr(), v.stride(0), v.stride(1),
+          qn ? q_w.data_ptr<float>() : nullptr,
+          kn ? k_w.data_ptr<float>() : nullptr, (float)eps,
+          (act_t*)k_cache.data_ptr(), (act_t*)v_cache.data_ptr(),
+          slot_mapping.data_ptr<int64_t>(), H, G, D, V, BS,
+          R > 0 ? positions.data_ptr<int64_t>() : nullptr,
+          R > 0 ? inv_freq.data_ptr<float>() : nullptr, R, (float)rot_mag,
+          unit_norm, interleaved,
+          blend ? (const act_t*)v_first.data_ptr() : nullptr,
+          blend ? v_first.stride(0) : 0, blend ? v_first.stride(1) : 0,
+          (float)v_lambda, lpr);
+      return;
+    }
     hipLaunchKernelGGL((qk_norm_cache_write_kernel<act_t>),
         dim3(T, H + 2 * G), dim3(64), 0, stream, (act_t*)q_out.data_ptr(),
         (const act_t*)q.data_ptr(), q.stride(0), q.stride(1),
