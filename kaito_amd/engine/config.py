@@ -108,6 +108,8 @@ class ModelConfig:
     # router outputs beyond num_experts that hand the input through
     # ("softmax_bias" routing); groups are formed over both
     moe_identity_experts: int = 0
+    # "softmax_bias" routing: the choice adds a per-expert correction
+    moe_choice_correction: bool = True
     n_group: int = 1                     # expert groups (V3: 8)
     topk_group: int = 1                  # groups kept per token (V3: 4)
     n_shared_experts: int = 0            # always-on experts (width = n*moe_ie)
@@ -155,6 +157,8 @@ class ModelConfig:
     residual_streams: int = 0
     # factor of every sub-layer's output in the residual sum
     residual_mult: float = 1.0
+    # factor of the logits, ahead of final_logit_softcap
+    logit_scale: float = 1.0
 
     @classmethod
     def from_hf_config(cls, cfg: dict, name: str = "") -> "ModelConfig":

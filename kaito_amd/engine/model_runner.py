@@ -231,6 +231,7 @@ class ModelRunner:
             meta.token_seq = torch.tensor(seq_of, dtype=torch.int32,
                                           device=dev)
             meta.ctx_lens = [c.start + c.length for c in chunks]
+            meta.ctx_starts = [c.start for c in chunks]
             if self.is_gpu and meta.max_seqlen >= 8:
                 # prompt portions: tile the chunks for the MFMA attention
                 # kernel (a step of single tokens keeps the decode kernel)

@@ -34,6 +34,10 @@ class MixerLayerBase(nn.Module):
                 out[type(m).__name__ + "." + k] = t
         return out
 
+    def slot_bytes(self) -> int:
+        """Bytes per state slot of the layer itself, beside its mixers'."""
+        return 0
+
     @staticmethod
     def _view(cache, m):
         pre = type(m).__name__ + "."
@@ -69,6 +73,11 @@ class HybridStackBase(nn.Module):
         """No position table: rotations, where a design has them, are
         computed from the position inside the kernels."""
 
+    def run_layers(self) -> List[MixerLayerBase]:
+        """Layers in execution order; one on shared weights appears once
+        per run, and every run has caches and states of its own."""
+        return list(self.layers)
+
     def stack_state(self, num_slots, device) -> Dict:
         """Per-sequence state that belongs to the stack rather than to a
         layer (slot-indexed tensors); handed to forward() as the entry
@@ -80,7 +89,8 @@ class HybridStackBase(nn.Module):
         page = 0
         slot = sum(t.element_size() * t[0].numel()
                    for t in self.stack_state(1, "cpu").values())
-        for layer in self.layers:
+        for layer in self.run_layers():
+            slot += layer.slot_bytes()
             for m in layer.mixers():
                 p, s = m.cache_bytes(block_size)
                 page += p
@@ -90,7 +100,7 @@ class HybridStackBase(nn.Module):
     def alloc_caches(self, num_blocks, block_size, num_slots,
                      device) -> List[Dict]:
         return [layer.alloc_cache(num_blocks, block_size, num_slots, device)
-                for layer in self.layers] \
+                for layer in self.run_layers()] \
             + [self.stack_state(num_slots, device)]
 
     def compute_logits(self, hidden: torch.Tensor) -> torch.Tensor:

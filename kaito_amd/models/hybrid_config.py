@@ -1,6 +1,6 @@
 """Per-layer specifications for hybrid stacks (recurrent, windowed and
 latent attention layers mixed in one model) and the config.json readers of
-the Gurapel, Pokulorn, Munerax, Lokedra and Vemenex designs.
+the Gurapel, Pokulorn, Munerax, Lokedra, Vemenex and Labirax designs.
 
 A homogeneous model is described by the flat ModelConfig fields; a hybrid
 one additionally carries `layer_specs`, one LayerSpec per layer, each
@@ -65,7 +65,8 @@ class MoESpec:
     scores the sum of its two best experts, only the `keep_groups` best
     groups are eligible; weights are the chosen scores times `scale`, not
     renormalised) or "softmax_bias" (softmax over all experts; the choice
-    adds a per-expert correction to the scores, the weights are the chosen
+    adds a per-expert correction to the scores (none with `correction`
+    off), the weights are the chosen
     scores without it, over their sum with `renorm`; with `groups` > 1 a
     group scores its largest corrected score; the last `identity` router
     outputs, beyond the `experts`, hand the input through and belong to
@@ -86,6 +87,7 @@ class MoESpec:
     limit: float = 0.0            # clamp of "clamped_glu"
     renorm: bool = False
     identity: int = 0
+    correction: bool = True
 
 
 @dataclass(frozen=True)
@@ -128,6 +130,14 @@ class RotarySpec:
 
 
 @dataclass(frozen=True)
+class QueryTempSpec:
+    """Query temperature growing with the position p: scores are scaled by
+    1 + coef * ln(floor((p + 1) / every) + 1)."""
+    coef: float
+    every: int
+
+
+@dataclass(frozen=True)
 class RotaryAttnSpec:
     """Softmax attention over the paged cache with short causal
     convolutions on q/k/v, per-head qk RMS norm (shared weight), partial
@@ -160,6 +170,12 @@ class RotaryAttnSpec:
     # normalisation over the keys
     sigmoid_scores: bool = False
     head_gate: bool = False       # sigmoid output gate, one number per head
+    qkv_bias: bool = False        # biases on the q/k/v projections only
+    # a learned bias per head and distance joins the (scaled) score;
+    # distances from `bias_max` on share one value (0 = none). The
+    # checkpoint holds it by buckets of distances (distance_bias_table)
+    bias_max: int = 0
+    q_temp: Optional[QueryTempSpec] = None
 
 
 @dataclass(frozen=True)
@@ -206,7 +222,9 @@ class LatentAttnSpec:
     denominator, a per-head sigmoid output gate, and `kv_from` = index of
     an earlier layer whose cached latent and rotated key this layer
     reads instead of projecting its own. `q_rank` > 0: queries are an
-    up-projection of an RMS-normed latent of that size."""
+    up-projection of an RMS-normed latent of that size. `window` > 0: a
+    query sees itself and window - 1 earlier keys. `value_gate`: the
+    output gate has a number per head and value dimension."""
     heads: int
     dim: int
     rot_dim: int
@@ -218,6 +236,8 @@ class LatentAttnSpec:
     gate: bool = False
     kv_from: Optional[int] = None
     q_rank: int = 0
+    window: int = 0
+    value_gate: bool = False
 
 
 @dataclass(frozen=True)
@@ -243,6 +263,18 @@ class HGRN2Spec:
     heads: int
     dim: int
     vdim: int
+
+
+@dataclass(frozen=True)
+class GLASpec:
+    """Gated linear attention with a decay per key channel: per head
+    S <- diag(alpha) S + k v^T, o = S^T q / sqrt(dim), alpha =
+    sigmoid(low-rank(h) + b)^(1/tau); o is RMS-normed over vdim with a
+    weight shared by the heads and multiplied by silu(W_g h)."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
 
 
 @dataclass(frozen=True)
@@ -288,6 +320,9 @@ class LayerSpec:
     # with `branch_scales`; feed-forward `moe` or none.
     # Vemenex — "attention" (sigmoid scores) and "attention_2" (unit sink,
     # head gate): RotaryAttnSpec; feed-forward `glu`, `moe` or none.
+    # Labirax — "gla": GLASpec; "latent_attention": LatentAttnSpec (window,
+    # value gate); "attention": RotaryAttnSpec (distance bias, query
+    # temperature); feed-forward `moe` or none.
     kind: str
     delta: Optional[DeltaRuleSpec] = None
     attn: Optional[WindowAttnSpec] = None
@@ -302,6 +337,10 @@ class LayerSpec:
     glu: Optional[GLUSpec] = None
     ddelta: Optional[DiagDeltaSpec] = None
     hgrn: Optional[HGRN2Spec] = None
+    gla: Optional[GLASpec] = None
+    # index of the layer whose weights this one runs on, with caches and
+    # states of its own (None = weights of its own)
+    weights_of: Optional[int] = None
 
 
 def _moe_spec(m) -> Optional[MoESpec]:
@@ -375,18 +414,22 @@ def layer_moe_config(cfg: ModelConfig, moe: MoESpec) -> ModelConfig:
     the 64-column tile of the fused grouped-GEMM kernels (which also keeps
     the vectorised activation kernel's alignment on the per-expert path);
     the loader zero-fills the extra gate/up rows and down columns, which
-    contribute exactly nothing (silu(0)·0 = 0)."""
-    ff = moe.ff
+    contribute exactly nothing (silu(0)·0 = 0). A gated shared expert is
+    rounded up to the activation kernel's 8 columns in the same way."""
+    ff, shared = moe.ff, moe.shared_ff
     if cfg.dtype == torch.bfloat16:
         ff = (ff + 63) // 64 * 64
+        if moe.act != "relu2":
+            shared = (shared + 7) // 8 * 8
     return dataclasses.replace(
         cfg, num_experts=moe.experts, num_experts_per_tok=moe.top,
         moe_intermediate_size=ff, moe_routing=moe.routing,
         moe_act="silu" if moe.act == "silu_glu" else moe.act,
         moe_bias=False, n_shared_experts=0,
-        moe_shared_intermediate_size=moe.shared_ff, n_group=moe.groups,
+        moe_shared_intermediate_size=shared, n_group=moe.groups,
         topk_group=moe.keep_groups, moe_norm_topk=moe.renorm,
         moe_identity_experts=moe.identity,
+        moe_choice_correction=moe.correction,
         routed_scaling_factor=moe.scale, moe_router_fp32=True,
         moe_act_limit=moe.limit)
 
@@ -730,5 +773,125 @@ def vemenex_model_config(cfg: dict, name: str = "",
         residual_streams=int(cfg["streams"]),
         residual_mult=float(cfg["residual_mult"]), residual_fp32=True,
         num_experts=moe.experts if moe else 0,
+        num_experts_per_tok=moe.top if moe else 0,
+        moe_intermediate_size=moe.ff if moe else 0, dtype=dtype)
+
+
+# ---- Labirax ------------------------------------------------------------------
+
+def distance_bias_table(rel: torch.Tensor, bias_max: int) -> torch.Tensor:
+    """Bias rows per bucket of distances, [B, heads], spread out to one value
+    per head and distance, [heads, bias_max + 1] f32. The lower half of the
+    buckets hold one distance each, the others grow logarithmically up to
+    bias_max; all larger distances share the last bucket."""
+    import math
+    n_buckets = rel.shape[0]
+    half = n_buckets // 2
+    if not 1 <= half < bias_max:
+        raise ValueError(f"distance bias: {n_buckets} buckets do not fit "
+                         f"distances up to {bias_max}")
+    rows = []
+    for n in range(bias_max + 1):
+        if n < half:
+            rows.append(n)
+            continue
+        up = math.floor(math.log(n / half) / math.log(bias_max / half)
+                        * (n_buckets - half))
+        rows.append(min(n_buckets - 1, half + up))
+    return rel.float()[torch.tensor(rows)].t().contiguous()
+
+
+def _labirax_ff(m) -> Optional[MoESpec]:
+    if m is None:
+        return None
+    if m.get("kind", "moe") != "moe":
+        raise ValueError(f"unsupported feed-forward kind {m.get('kind')!r}")
+    r = m["router"]
+    moe = MoESpec(
+        experts=int(r["experts"]), top=int(r["top"]),
+        ff=int(m["expert"]["ff"]), routing="softmax_bias", renorm=True,
+        correction=False, shared_ff=int((m.get("shared") or {}).get("ff", 0)))
+    if not 1 <= moe.top <= moe.experts:
+        raise ValueError(f"router: top {moe.top} of {moe.experts} experts")
+    return moe
+
+
+def _labirax_layer(entry: dict) -> LayerSpec:
+    kind, mx = entry["type"], entry["mixer"]
+    moe = _labirax_ff(entry.get("mlp"))
+    if kind == "gla":
+        return LayerSpec(kind, gla=GLASpec(
+            heads=int(mx["heads"]), dim=int(mx["dim"]), vdim=int(mx["vdim"]),
+            tau=float(mx["tau"])), moe=moe)
+    if kind == "latent_attention":
+        rot = mx["rot"]
+        if int(rot["dims"]) != int(mx["rot_dim"]):
+            raise ValueError("the rotated key part is rotated whole")
+        return LayerSpec(kind, latent=LatentAttnSpec(
+            heads=int(mx["heads"]), dim=int(mx["dim"]),
+            rot_dim=int(mx["rot_dim"]), vdim=int(mx["vdim"]),
+            kv_rank=int(mx["kv_rank"]), scale=float(mx["scale"]),
+            rot=RotarySpec(dims=int(rot["dims"]), base=float(rot["base"])),
+            q_rank=int(mx["q_rank"]),
+            window=int((mx.get("mask") or {}).get("size", 0)),
+            value_gate=True), moe=moe)
+    if kind == "attention":
+        qt = mx.get("q_temp")
+        return LayerSpec(kind, rattn=RotaryAttnSpec(
+            heads=int(mx["heads"]), kv_heads=int(mx["kv_heads"]),
+            dim=int(mx["dim"]), vdim=int(mx["vdim"]),
+            scale=float(mx["scale"]), qk_norm=False, qkv_bias=True,
+            bias_max=int(mx["bias_max"]),
+            q_temp=QueryTempSpec(coef=float(qt["coef"]),
+                                 every=int(qt["every"])) if qt else None),
+            moe=moe)
+    raise ValueError(f"unknown layer type {kind!r}")
+
+
+def is_labirax_config(cfg: dict) -> bool:
+    return cfg.get("architecture") == "Labirax"
+
+
+def labirax_model_config(cfg: dict, name: str = "",
+                         dtype: torch.dtype = torch.bfloat16) -> ModelConfig:
+    """config.json of a Labirax checkpoint → ModelConfig (every size, the
+    layer order, shared weights and every per-model constant come from the
+    file). The design has no position table, so its length limit is the
+    engine's."""
+    entries = cfg["layers"]
+    specs = []
+    for i, e in enumerate(entries):
+        spec, src = _labirax_layer(e), e.get("weights_of")
+        seen, home = {i}, None
+        while src is not None:          # down to the layer with the tensors
+            src = int(src)
+            if not 0 <= src < len(entries) or src in seen:
+                raise ValueError(f"layer {i}: weights_of does not lead to a "
+                                 "layer with weights")
+            if _labirax_layer(entries[src]) != spec:
+                raise ValueError(f"layer {i} differs from layer {src}, whose "
+                                 "weights it runs on")
+            seen.add(src)
+            home, src = src, entries[src].get("weights_of")
+        specs.append(dataclasses.replace(spec, weights_of=home))
+    width = int(cfg["width"])
+    att = next((s.rattn for s in specs if s.rattn is not None), None)
+    moe = next((s.moe for s in specs if s.moe is not None), None)
+    return ModelConfig(
+        name=name or "labirax", arch="labirax", layer_specs=tuple(specs),
+        hidden_size=width, num_layers=len(specs),
+        num_heads=att.heads if att else 1,
+        num_kv_heads=att.kv_heads if att else 1,
+        head_dim=att.dim if att else width,
+        intermediate_size=moe.ff if moe else width,
+        vocab_size=int(cfg["vocab"]),
+        max_position=int(cfg.get("max_positions",
+                                 POKULORN_DEFAULT_MAX_POSITION)),
+        rms_eps=float(cfg["norm"]["eps"]), norm_type="layernorm",
+        sandwich_norms=True,
+        embed_scale=float(cfg["embedding"].get("scale", 1.0)),
+        logit_scale=float(cfg.get("logit_scale", 1.0)),
+        final_logit_softcap=float(cfg.get("logit_softcap") or 0.0),
+        residual_fp32=True, num_experts=moe.experts if moe else 0,
         num_experts_per_tok=moe.top if moe else 0,
         moe_intermediate_size=moe.ff if moe else 0, dtype=dtype)

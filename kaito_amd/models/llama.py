@@ -50,6 +50,8 @@ class AttnMetadata:
     # host copy of each chunk's context length after the step (start +
     # chunk length), for ops that size step-local buffers by it
     ctx_lens: Optional[list] = None
+    # host copy of seq_starts, kept beside ctx_lens
+    ctx_starts: Optional[list] = None
     # values one layer of a step leaves for later layers of the same step
     # (the model's forward sets an empty dict)
     layer_shared: Optional[dict] = None

@@ -34,6 +34,8 @@ def load_safetensors_weights(model, path: str,
         return load_lokedra_weights(model, path)
     if getattr(model.cfg, "arch", "llama") == "vemenex":
         return load_vemenex_weights(model, path)
+    if getattr(model.cfg, "arch", "llama") == "labirax":
+        return load_labirax_weights(model, path)
     from safetensors.torch import safe_open
 
     cfg = model.cfg
@@ -576,11 +578,13 @@ def load_lokedra_weights(model, path: str) -> None:
 
 
 def _load_routed(ck, mlp, fp: str) -> None:
-    """Router, choice correction and gated experts under prefix fp (experts
-    zero-filled up to the kernels' tile width)."""
+    """Router, choice correction (where there is one), gated experts
+    (zero-filled up to the kernels' tile width) and shared expert under
+    prefix fp."""
     get, put = ck.get, ck.put
     put(mlp.gate, get(fp + "router").float())
-    put(mlp.e_score_correction_bias, get(fp + "correction").float())
+    if mlp.e_score_correction_bias is not None:
+        put(mlp.e_score_correction_bias, get(fp + "correction").float())
     ie = mlp.ie_local
     with torch.no_grad():
         mlp.w_gate_up.zero_()
@@ -592,6 +596,13 @@ def _load_routed(ck, mlp, fp: str) -> None:
             mlp.w_gate_up[e, :ff].copy_(g.to(dt))
             mlp.w_gate_up[e, ie:ie + ff].copy_(u.to(dt))
             mlp.w_down[e, :, :ff].copy_(d.to(dt))
+    if mlp.w_shared_gate_up is not None:
+        pad = torch.nn.functional.pad
+        g, u, d = (get(f"{fp}shared.{n}") for n in ("gate", "up", "down"))
+        more = mlp.sie_local - g.shape[0]       # zero rows and columns
+        put(mlp.w_shared_gate_up, torch.cat(
+            [pad(g, (0, 0, 0, more)), pad(u, (0, 0, 0, more))], 0))
+        put(mlp.w_shared_down, pad(d, (0, more)))
 
 
 def load_vemenex_weights(model, path: str) -> None:
@@ -636,4 +647,60 @@ def load_vemenex_weights(model, path: str) -> None:
             put(layer.mlp.down, get(fp + "down"))
         elif layer.spec.moe is not None:
             _load_routed(ck, layer.mlp, fp)
+    ck.warn_unused()
+
+
+def load_labirax_weights(model, path: str) -> None:
+    """Labirax checkpoint (flat tensor names, `l<i>.` per layer that has
+    weights, mixer tensors under `.mix.`, feed-forward under `.mlp.`, linear
+    weights [out, in]) → LabiraxForCausalLM. Fuses each mixer's input
+    projections, spreads the distance bias out per distance, sizes the decay
+    bottleneck by the checkpoint's tensors, stacks the experts and widens
+    norms, biases and the router to f32."""
+    from .hybrid_config import distance_bias_table
+    ck = _FlatCheckpoint(path)
+    get, put = ck.get, ck.put
+    cat = torch.cat
+
+    def put_norm(norm, name):
+        put(norm.weight, get(name).float())
+        put(norm.bias, get(name + ".b").float())
+
+    put(model.embed_tokens.weight, get("embed"))
+    put_norm(model.norm, "final.norm")
+    put(model.lm_head, get("head"))
+    for i, layer in zip(model.layer_ids, model.layers):
+        pre, mp = f"l{i}.", f"l{i}.mix."
+        m, kind = layer.mixer, layer.spec.kind
+        for name, norm in layer.norms().items():
+            put_norm(norm, pre + name)
+        if kind == "gla":
+            put(m.in_proj, cat([get(mp + n) for n in "qkvg"], 0))
+            a1 = get(mp + "a1")
+            if a1.shape[0] != m.decay_rank:
+                m.set_decay_rank(int(a1.shape[0]))
+            put(m.a1, a1)
+            put(m.a2, get(mp + "a2").float().t())
+            put(m.a_bias, get(mp + "a2.b").float())
+            put(m.out_norm, get(mp + "norm").float())
+        elif kind == "latent_attention":
+            w_in = cat([get(mp + n) for n in ("dq", "g", "dkv")], 0)
+            if w_in.shape[0] != m.in_rows:
+                raise ValueError(f"{mp}: projection rows {w_in.shape[0]} vs "
+                                 f"{m.in_rows} from the config")
+            put(m.in_proj, torch.nn.functional.pad(
+                w_in, (0, 0, 0, m.in_proj.shape[0] - m.in_rows)))
+            put(m.q_norm, get(mp + "dq.norm").float())
+            put(m.w_uq, get(mp + "uq"))
+            put(m.kv_norm, get(mp + "dkv.norm").float())
+            put(m.w_uk, get(mp + "uk"))
+            put(m.w_uv, get(mp + "uv"))
+        else:
+            put(m.qkv_proj, cat([get(mp + n) for n in "qkv"], 0))
+            put(m.qkv_bias, cat([get(mp + n + ".b") for n in "qkv"], 0))
+            put(m.dist_bias, distance_bias_table(get(mp + "rel"),
+                                                 m.spec.bias_max))
+        put(m.o_proj, get(mp + "o"))
+        if layer.mlp is not None:
+            _load_routed(ck, layer.mlp, pre + "mlp.")
     ck.warn_unused()

@@ -136,23 +136,8 @@ class LokedraForCausalLM(HybridStackBase):
         """The embedding table itself (without the input scale)."""
         return self.embed_tokens.weight
 
-    # every run of a layer keeps its own cache and state
-    def cache_bytes(self, block_size: int):
-        page = slot = 0
-        for li, _ in self.runs:
-            layer = self.layers[li]
-            slot += layer.slot_bytes()
-            for m in layer.mixers():
-                p, s = m.cache_bytes(block_size)
-                page += p
-                slot += s
-        return page, slot
-
-    def alloc_caches(self, num_blocks, block_size, num_slots,
-                     device) -> List[Dict]:
-        return [self.layers[li].alloc_cache(num_blocks, block_size,
-                                            num_slots, device)
-                for li, _ in self.runs]
+    def run_layers(self):
+        return [self.layers[li] for li, _ in self.runs]
 
     def decode_graph_capturable(self) -> bool:
         """True when no decode-step op reads device data on the host: the

@@ -4,10 +4,12 @@ state space, softmax attention over the paged cache in two flavours
 (distance penalty without rotation; convolutions + rotation + window
 with kept first tokens or a chunked mask + sink, optionally with the
 keys as values, optionally with sigmoid weights in place of the softmax
-and a gate per head), latent attention (one low-rank latent per token in the
+and a gate per head, optionally with a learned distance bias and a query
+temperature), latent attention (one low-rank latent per token in the
 cache, optionally borrowed from an earlier layer, optionally with
-low-rank queries), the generalized delta rule with per-channel decay, and
-gated linear attention with a tied write gate (HGRN2). Each is a self-contained module parameterised by its spec
+low-rank queries, optionally windowed), the generalized delta rule with per-channel decay, and
+gated linear attention with a tied write gate (HGRN2) or a low-rank decay
+(GLA). Each is a self-contained module parameterised by its spec
 (models/hybrid_config.py), so a design picks and combines them freely.
 
 All follow the same calling convention:
@@ -35,7 +37,7 @@ import torch.nn.functional as F
 
 from .. import ops
 from .hybrid_config import (DeltaRuleSpec, DenseFFSpec, DiagDeltaSpec,
-                            GLUSpec, HGRN2Spec, LatentAttnSpec,
+                            GLASpec, GLUSpec, HGRN2Spec, LatentAttnSpec,
                             MLSTMSpec, RGLRUSpec, RotaryAttnSpec, SSDSpec,
                             WindowAttnSpec)
 
@@ -243,7 +245,9 @@ class RotaryWindowAttention(nn.Module):
     projections may carry biases; the heads' outputs may be gated by
     sigmoid of a fourth projection, per value dimension or per head. The
     norm of q and k may be a plain one behind the rotation, and a key's
-    weight may be sigmoid(score + a per-head bias) instead of a softmax."""
+    weight may be sigmoid(score + a per-head bias) instead of a softmax.
+    A learned bias per head and distance may join the scores, and the
+    queries may carry a temperature that grows with their position."""
 
     def __init__(self, hidden: int, spec: RotaryAttnSpec, dtype,
                  norm_eps: float):
@@ -266,7 +270,7 @@ class RotaryWindowAttention(nn.Module):
         self.qkv_proj = _p(-(-self.in_rows // 8) * 8 if s.head_gate
                            else self.in_rows, hidden, dtype=dtype)
         self.qkv_bias = _p(self.qkv_proj.shape[0], dtype=dtype) \
-            if s.bias else None
+            if s.bias or s.qkv_bias else None
         self.o_bias = _p(hidden, dtype=dtype) if s.bias else None
         self.conv_weight = _p(self.conv_ch, s.conv_taps, dtype=torch.float32) \
             if s.conv_taps > 0 else None
@@ -291,6 +295,8 @@ class RotaryWindowAttention(nn.Module):
                 s.heads, dtype=torch.float32), persistent=False)
         else:
             self.sinks = _p(s.heads, dtype=torch.float32) if s.sink else None
+        self.dist_bias = _p(s.heads, s.bias_max + 1, dtype=torch.float32) \
+            if s.bias_max > 0 else None
         # blend weight of the first value-mixing layer's values; the first
         # such layer of a stack never reads it
         self.v_lambda = 0.0
@@ -357,7 +363,11 @@ class RotaryWindowAttention(nn.Module):
                                  keep_first=s.keep_first, sinks=self.sinks,
                                  chunk=s.chunk, sigmoid_bias=self.score_bias,
                                  gate=p[:, self.conv_ch:self.in_rows]
-                                 if s.head_gate else None)
+                                 if s.head_gate else None,
+                                 dist_bias=self.dist_bias,
+                                 temp_coef=s.q_temp.coef if s.q_temp else 0.0,
+                                 temp_every=s.q_temp.every if s.q_temp
+                                 else 1)
         o = o.reshape(T, self.o_size)
         if s.gate:
             o = ops.sigmoid_mul(o, p[:, self.conv_ch:])
@@ -498,8 +508,8 @@ class LatentAttention(nn.Module):
     `rot_dim` dims shared by all heads; head h's key is [W_uk,h c | rotated
     part] and its value W_uv,h c. Queries carry `dim` unrotated and
     `rot_dim` rotated dims per head. Options: per-head sink in the softmax
-    denominator, per-head sigmoid output gate read from the mixer input,
-    queries through an RMS-normed latent of their own (spec.q_rank), the
+    denominator, sigmoid output gate read from the mixer input (per head
+    or per value dimension), a sliding window, queries through an RMS-normed latent of their own (spec.q_rank), the
     rotation pairing neighbours (2i, 2i + 1) and carrying interpolated
     frequencies with a magnitude. With spec.kv_from set the mixer has no down-projection and reads the
     cache of the layer it names (the caller passes that layer's cache).
@@ -524,7 +534,9 @@ class LatentAttention(nn.Module):
             and s.rot_dim % 2 == 0
         self.own_kv = s.kv_from is None
         self.q_size = s.heads * (s.dim + s.rot_dim)
-        self.g_size = s.heads if s.gate else 0
+        assert not (s.gate and s.value_gate)
+        self.g_size = s.heads * s.vdim if s.value_gate \
+            else (s.heads if s.gate else 0)
         self.row = s.kv_rank + s.rot_dim
         # fused input projection, rows [q (or its latent) | gate | latent +
         # rotated key], zero rows up to a multiple of 8 so that output
@@ -545,6 +557,9 @@ class LatentAttention(nn.Module):
             freq, dtype=torch.float64).float(), persistent=False)
         self.sinks = _p(s.heads, dtype=torch.float32) if s.sink else None
         self.o_proj = _p(hidden, s.heads * s.vdim, dtype=dtype)
+        # W_uv per head as [rank, vdim] for the batched product, made when
+        # first needed and again after the weights change
+        self._uv_t, self._uv_src = None, None
 
     def alloc_cache(self, num_blocks, block_size, num_slots, device) -> Dict:
         if not self.own_kv:
@@ -557,6 +572,15 @@ class LatentAttention(nn.Module):
             return 0, 0
         esz = torch.empty(0, dtype=self.dtype).element_size()
         return block_size * self.row * esz, 0
+
+    def _uv_by_head(self):
+        src = (self.w_uv.data_ptr(), self.w_uv._version)
+        if self._uv_src != src:
+            s = self.spec
+            self._uv_t = self.w_uv.detach().view(
+                s.heads, s.vdim, s.kv_rank).transpose(1, 2).contiguous()
+            self._uv_src = src
+        return self._uv_t
 
     def _expanded_ok(self, x, meta) -> bool:
         s = self.spec
@@ -571,7 +595,7 @@ class LatentAttention(nn.Module):
         T, H, D = x.size(0), s.heads, s.dim
         p = F.linear(x, self.in_proj)
         if s.q_rank > 0:
-            cq = ops.rms_norm_cast(p[:, :s.q_rank].contiguous(), self.q_norm,
+            cq = ops.rms_norm_cast(p[:, :s.q_rank], self.q_norm,
                                    self.norm_eps, self.dtype)
             q = F.linear(cq, self.w_uq).unflatten(-1, (H, D + s.rot_dim))
         else:
@@ -595,13 +619,14 @@ class LatentAttention(nn.Module):
             qf = torch.cat([qc.transpose(0, 1), qr[..., D:]], -1)
             oc = ops.latent_attention(qf, kv, meta.block_tables,
                                       meta.token_seq, positions, s.scale,
-                                      s.kv_rank, self.sinks)     # [T, H, r]
+                                      s.kv_rank, self.sinks,
+                                      s.window)                  # [T, H, r]
             o = torch.bmm(oc.transpose(0, 1),
-                          self.w_uv.view(H, s.vdim, s.kv_rank)
-                          .transpose(1, 2)).transpose(0, 1)
+                          self._uv_by_head()).transpose(0, 1)
         o = o.reshape(T, H * s.vdim)
-        if s.gate:
-            o = ops.sigmoid_mul(o, p[:, self.q_rows:self.q_rows + H])
+        if self.g_size:
+            o = ops.sigmoid_mul(o, p[:, self.q_rows:self.q_rows
+                                     + self.g_size])
         return F.linear(o, self.o_proj)
 
     def _expanded(self, qr, kv, meta):
@@ -611,13 +636,17 @@ class LatentAttention(nn.Module):
         H, D, R, V = s.heads, s.dim, s.rot_dim, s.vdim
         Dp = qr.size(2)                 # queries arrive zero-padded
         Vp = next(v for v in ops.WINDOW_MFMA_VSIZES if v >= V)
-        lat, tables = ops.latent_gather(kv, meta.block_tables, meta.ctx_lens)
+        first = [max(0, n - s.window + 1) for n in meta.ctx_starts] \
+            if s.window > 0 else None
+        lat, tables = ops.latent_gather(kv, meta.block_tables, meta.ctx_lens,
+                                        first)
         k_s, v_s = ops.latent_expand(
             F.linear(lat[:, :s.kv_rank], self.w_uk),
             F.linear(lat[:, :s.kv_rank], self.w_uv), lat, H, D, V, s.kv_rank,
             Dp, Vp, kv.size(1))
         o = ops.window_attention(
             qr, k_s, v_s, tables, meta.token_seq, None, s.scale,
+            window=s.window,
             tiles=(meta.tile_seq, meta.tile_qbase, meta.cu_seqlens,
                    meta.seq_starts), sinks=self.sinks)
         return o[..., :V]
@@ -741,4 +770,65 @@ class HGRN2Mixer(nn.Module):
             self.lower, self.out_norm, cache["ssm"], meta.cu_seqlens,
             meta.state_slots, meta.seq_starts, self.norm_eps,
             f_bias=self.f_bias)
+        return F.linear(o, self.o_proj)
+
+
+class GLAMixer(nn.Module):
+    """Gated linear attention with a decay per key channel: per head S <-
+    diag(alpha) S + k v^T, o = S^T q / sqrt(dim), alpha = sigmoid(W2 (W1 x)
+    + b)^(1/tau) (alpha scales state rows, which are indexed like k). o is
+    RMS-normed over vdim with a weight shared by the heads, multiplied by
+    silu(W_g x) and projected out. q, k, v and the gate come from one
+    activation-dtype projection; the decay's bottleneck W1 x stays f32, its
+    up-projection W2 is part of the scan kernel (f32)."""
+
+    def __init__(self, hidden: int, spec: GLASpec, dtype, norm_eps: float,
+                 decay_rank: int = 16):
+        super().__init__()
+        self.spec, self.dtype, self.norm_eps = spec, dtype, norm_eps
+        self.hidden = hidden
+        s = spec
+        self.n_q = s.heads * s.dim
+        self.n_v = s.heads * s.vdim
+        # fused input projection, rows [q | k | v | gate]
+        self.in_proj = _p(2 * self.n_q + 2 * self.n_v, hidden, dtype=dtype)
+        self.a_bias = _p(self.n_q, dtype=torch.float32)
+        self.out_norm = _p(s.vdim, dtype=torch.float32)
+        self.o_proj = _p(hidden, self.n_v, dtype=dtype)
+        self.set_decay_rank(decay_rank)
+
+    def set_decay_rank(self, rank: int):
+        """(Re)create the low-rank decay path for a bottleneck of `rank`
+        (a checkpoint's tensor shapes decide it)."""
+        dev = self.in_proj.device
+        self.decay_rank = rank
+        self.a1 = nn.Parameter(torch.empty(
+            rank, self.hidden, dtype=self.dtype, device=dev),
+            requires_grad=False)
+        self.a2 = nn.Parameter(torch.empty(          # [in, out]
+            rank, self.n_q, dtype=torch.float32, device=dev),
+            requires_grad=False)
+
+    def alloc_cache(self, num_blocks, block_size, num_slots, device) -> Dict:
+        s = self.spec
+        return {"ssm": torch.zeros(num_slots, s.heads, s.dim, s.vdim,
+                                   dtype=torch.float32, device=device)}
+
+    def cache_bytes(self, block_size: int):
+        s = self.spec
+        return 0, s.heads * s.dim * s.vdim * 4
+
+    def forward(self, x, positions, cache, meta):
+        s = self.spec
+        p = F.linear(x, self.in_proj)
+        low = ops.linear_f32(x, self.a1)
+        nq, nv = self.n_q, self.n_v
+        qk, vg = (s.heads, s.dim), (s.heads, s.vdim)
+        o = ops.gla_scan(
+            p[:, :nq].unflatten(-1, qk), p[:, nq:2 * nq].unflatten(-1, qk),
+            p[:, 2 * nq:2 * nq + nv].unflatten(-1, vg),
+            p[:, 2 * nq + nv:].unflatten(-1, vg), low, self.a2, self.a_bias,
+            s.tau, s.dim ** -0.5, self.out_norm, cache["ssm"],
+            meta.cu_seqlens, meta.state_slots, meta.seq_starts,
+            self.norm_eps)
         return F.linear(o, self.o_proj)

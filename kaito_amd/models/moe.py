@@ -89,7 +89,10 @@ class MoEMLP(nn.Module):
         self.act_limit = float(cfg.moe_act_limit) \
             if cfg.moe_act == "clamped_glu" else 7.0
         # per-expert selection bias (deepseek-v3 noaux_tc; softmax_bias)
-        if cfg.moe_routing in ("noaux_tc", "softmax_bias"):
+        self.e_score_correction_bias = None
+        if cfg.moe_routing == "noaux_tc" or (
+                cfg.moe_routing == "softmax_bias"
+                and cfg.moe_choice_correction):
             self.e_score_correction_bias = nn.Parameter(
                 torch.empty(self.n_route, dtype=torch.float32),
                 requires_grad=False)
@@ -192,9 +195,11 @@ class MoEMLP(nn.Module):
     import os as _os
     FUSED_MAX_TOKENS = int(_os.environ.get("KAITO_MOE_FUSED_MAX", "4096"))
 
-    def forward(self, x: torch.Tensor,
-                keep_f32: bool = False) -> torch.Tensor:
-        """keep_f32: the routed sum is returned as accumulated, in f32."""
+    def forward(self, x: torch.Tensor, keep_f32: bool = False,
+                split_shared: bool = False):
+        """keep_f32: the routed sum is returned as accumulated, in f32.
+        split_shared: returns (routed sum, the shared expert's output or
+        None) for a caller that adds them itself."""
         T, H = x.shape
         sorted_tok, gates, offsets, w_id = self._route(x)
         # the routed sum starts from the identity experts' share
@@ -212,11 +217,17 @@ class MoEMLP(nn.Module):
         else:
             self._forward_loop(x, sorted_tok, gates, offsets, out32)
         out = out32 if keep_f32 else out32.to(x.dtype)
+        shared = None
         if self.w_shared_gate_up is not None:   # deepseek shared experts
             h1 = torch.nn.functional.linear(x, self.w_shared_gate_up)
-            out = out + torch.nn.functional.linear(
+            shared = torch.nn.functional.linear(
                 ops.silu_and_mul(h1) if self.gated else ops.relu2(h1),
                 self.w_shared_down)
+        if split_shared:
+            assert get_state().tp_size == 1
+            return out, shared
+        if shared is not None:
+            out = out + shared
         if get_state().tp_size > 1:
             out = tp_all_reduce(out)
         return out

@@ -28,6 +28,7 @@ MODEL_CLASSES: Dict[str, str] = {
     "munerax": "kaito_amd.models.munerax:MuneraxForCausalLM",
     "lokedra": "kaito_amd.models.lokedra:LokedraForCausalLM",
     "vemenex": "kaito_amd.models.vemenex:VemenexForCausalLM",
+    "labirax": "kaito_amd.models.labirax:LabiraxForCausalLM",
 }
 
 
@@ -46,8 +47,9 @@ def config_from_checkpoint(cfg_json: dict, name: str = "",
     """config.json dict → ModelConfig, choosing the reader by the file's
     own architecture tag."""
     from .hybrid_config import (gurapel_model_config, is_gurapel_config,
-                                is_lokedra_config, is_munerax_config,
-                                is_pokulorn_config, is_vemenex_config,
+                                is_labirax_config, is_lokedra_config,
+                                is_munerax_config, is_pokulorn_config,
+                                is_vemenex_config, labirax_model_config,
                                 lokedra_model_config, munerax_model_config,
                                 pokulorn_model_config, vemenex_model_config)
     kw = {"dtype": dtype} if dtype is not None else {}
@@ -61,6 +63,8 @@ def config_from_checkpoint(cfg_json: dict, name: str = "",
         return lokedra_model_config(cfg_json, name=name, **kw)
     if is_vemenex_config(cfg_json):
         return vemenex_model_config(cfg_json, name=name, **kw)
+    if is_labirax_config(cfg_json):
+        return labirax_model_config(cfg_json, name=name, **kw)
     cfg = ModelConfig.from_hf_config(cfg_json, name=name)
     if dtype is not None:
         import dataclasses
@@ -514,3 +518,31 @@ def _tiny_vemenex() -> ModelConfig:
 
 
 register(_tiny_vemenex())
+
+
+def _tiny_labirax() -> ModelConfig:
+    """A small sandwich-normed stack (gated linear attention, windowed
+    latent attention, attention with a distance bias, routed experts, two
+    layers on shared weights) for tests and smoke runs (random weights)."""
+    from .hybrid_config import labirax_model_config
+    moe = {"kind": "moe", "expert": {"ff": 48}, "shared": {"ff": 80},
+           "router": {"experts": 6, "top": 2}}
+    att = {"type": "attention", "mlp": moe, "mixer": {
+        "heads": 4, "kv_heads": 2, "dim": 16, "vdim": 24, "bias_max": 100,
+        "scale": 0.25, "q_temp": {"coef": 0.2, "every": 64}}}
+    gla = {"type": "gla", "mlp": moe, "mixer": {
+        "heads": 3, "dim": 16, "vdim": 24, "tau": 8.0}}
+    lat = {"type": "latent_attention", "mlp": None, "mixer": {
+        "heads": 3, "dim": 16, "rot_dim": 8, "vdim": 24, "kv_rank": 40,
+        "q_rank": 56, "mask": {"size": 30}, "scale": 0.2,
+        "rot": {"base": 10000.0, "dims": 8}}}
+    return labirax_model_config({
+        "architecture": "Labirax", "embedding": {"scale": 2.0},
+        "layers": [att, gla, lat, dict(att, weights_of=0),
+                   dict(gla, weights_of=1)],
+        "logit_scale": 1.5, "logit_softcap": 20.0, "norm": {"eps": 1e-5},
+        "vocab": 512, "width": 192, "max_positions": 1024},
+        name="tiny-labirax-test")
+
+
+register(_tiny_labirax())

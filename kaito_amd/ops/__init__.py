@@ -37,13 +37,15 @@ for _g, _names in {
             "qk_norm_cache_write window_attention window_attention_tiles "
             "post_norm_residual rms_norm_cast residual_add_norm "
             "scaled_residual_add_norm token_shift "
-            "clamped_glu sigmoid_mul gelu_glu relu_glu relu2"),
+            "clamped_glu sigmoid_mul gelu_glu relu_glu relu2 "
+            "scaled_softcap"),
     "latent": ("bigram_embed latent_rope_cache_write latent_attention "
                "latent_expand"),
     "delta": "gated_delta_rule rglru_scan",
-    "diag": "diag_delta_rule hgrn2_scan",
+    "diag": "diag_delta_rule hgrn2_scan gla_scan",
     "decay": "mlstm_scan ssd_scan",
     "streams": "stream_mix_norm stream_embed",
+    "lnorm": "layer_norm_cast embed_layer_norm sandwich_norm_residual",
 }.items():
     for _n in _names.split():
         _OP_GROUP[_n] = _g
@@ -337,7 +339,7 @@ MOE_ROUTE_MAX = (1024, 64, 64)      # router outputs, chosen, groups
 def moe_route(logits, correction, top: int, n_real: int, groups: int = 1,
               keep: int = 1, renorm: bool = False, scale: float = 1.0):
     """Expert choice from f32 router logits [T, N]: scores s = softmax; the
-    choice adds `correction` [N] f32; outputs form `groups` equal groups of
+    choice adds `correction` [N] f32 (None: nothing); outputs form `groups` equal groups of
     neighbours scored by their largest choice, of which the `keep` best
     stay eligible; the `top` largest eligible choices are taken. Weights
     are s (without the correction), over their sum + 1e-20 with `renorm`,
@@ -348,8 +350,8 @@ def moe_route(logits, correction, top: int, n_real: int, groups: int = 1,
         f32 = dict(dtype=torch.float32, device=logits.device)
         topi = torch.empty(T, top, dtype=torch.int32, device=logits.device)
         topw, w_id = torch.empty(T, top, **f32), torch.empty(T, **f32)
-        _K.moe_route(topi, topw, w_id, logits, correction, n_real, groups,
-                     keep, renorm, scale)
+        _K.moe_route(topi, topw, w_id, logits, _none(correction, logits),
+                     n_real, groups, keep, renorm, scale)
         return topi, topw, w_id
     return torch_ref.moe_route(logits, correction, top, n_real, groups, keep,
                                renorm, scale)
@@ -518,7 +520,8 @@ def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
                      scale: float, softcap: float = 0.0, r1=None, r2=None,
                      window: int = 0, tiles=None, keep_first: int = 0,
                      sinks=None, chunk: int = 0, sigmoid_bias=None,
-                     gate=None):
+                     gate=None, dist_bias=None, temp_coef: float = 0.0,
+                     temp_every: int = 1):
     """Causal attention of query rows [T, H, D] over the paged cache (key
     size D, value size V may differ). A query at position i sees keys
     j <= i with i - j < window or j < keep_first (window <= 0: all), or,
@@ -529,6 +532,9 @@ def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
     `sigmoid_bias` [H] f32 there is no softmax: a visible key's weight is
     sigmoid(score + bias), not normalised over the keys. `gate` [T, H]
     (row stride free) multiplies every head's output by its sigmoid.
+    `dist_bias` [H, N] f32: entry min(i - j, N - 1) of the head's row is
+    added to the score. `temp_coef` scales the products of the query at
+    position i by 1 + temp_coef*ln((i + 1) // temp_every + 1).
     Returns [T, H, V].
 
     `tiles` = (tile_seq, tile_qbase, cu_seqlens, seq_starts) describes the
@@ -548,18 +554,21 @@ def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
                 out, q, k_cache, v_cache, block_tables, tile_seq, tile_qbase,
                 cu, starts, scale, softcap, _none(r1, q), _none(r2, q),
                 window, keep_first, _none(sinks, q), chunk,
-                _none(sigmoid_bias, q), _none(gate, q))
+                _none(sigmoid_bias, q), _none(gate, q), _none(dist_bias, q),
+                temp_coef, temp_every)
             return out
         _K.window_attention(out, q, k_cache, v_cache, block_tables, token_seq,
                             positions, scale, softcap, _none(r1, q),
                             _none(r2, q), window, keep_first,
                             _none(sinks, q), chunk, _none(sigmoid_bias, q),
-                            _none(gate, q))
+                            _none(gate, q), _none(dist_bias, q), temp_coef,
+                            temp_every)
         return out
     return torch_ref.window_attention(q, k_cache, v_cache, block_tables,
                                       token_seq, positions, scale, softcap,
                                       r1, r2, window, keep_first, sinks,
-                                      chunk, sigmoid_bias, gate)
+                                      chunk, sigmoid_bias, gate, dist_bias,
+                                      temp_coef, temp_every)
 
 
 def build_query_tiles(chunk_lens, device):
@@ -591,7 +600,8 @@ def post_norm_residual(x32, y, w, eps: float, out_dtype, y2=None, w_y=None,
 
 
 def rms_norm_cast(x, weight, eps: float, out_dtype):
-    """RMS norm of f32 or bf16 rows with an f32 weight → out_dtype."""
+    """RMS norm of f32 or bf16 rows (row stride free) with an f32 weight
+    → out_dtype."""
     if x.is_cuda:
         out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
         _K.rms_norm_cast(out, x, weight, eps)
@@ -763,26 +773,29 @@ def latent_rope_cache_write(q, dkv, norm_w, eps: float, cache, slot_mapping,
 
 
 def latent_attention(q, cache, block_tables, token_seq, positions,
-                     scale: float, rank: int, sinks=None):
+                     scale: float, rank: int, sinks=None, window: int = 0):
     """Causal attention of latent-space queries [T, H, rank + P] over the
     paged latent cache [blocks, block_size, rank + P]: score = q . row *
-    scale over rows 0..position of the row's sequence, optional per-head
+    scale over rows 0..position of the row's sequence (with window > 0 the
+    last `window` of them), optional per-head
     sinks in the denominator, output = weighted sum of the rows' first
     `rank` dims, [T, H, rank]. One pass over the cache serves all heads."""
     if q.is_cuda:
         out = torch.empty(q.size(0), q.size(1), rank, dtype=q.dtype,
                           device=q.device)
         _K.latent_attention(out, q, cache, block_tables, token_seq,
-                            positions, scale, _none(sinks, q))
+                            positions, scale, _none(sinks, q), window)
         return out
     return torch_ref.latent_attention(q, cache, block_tables, token_seq,
-                                      positions, scale, rank, sinks)
+                                      positions, scale, rank, sinks, window)
 
 
-def latent_gather(cache, block_tables, ctx_lens):
+def latent_gather(cache, block_tables, ctx_lens, first_keys=None):
     """Whole pages of the step's sequences out of the paged latent cache:
     chunk b's first ceil(ctx_lens[b] / block_size) pages, in block-table
-    order. Returns (rows [pages * block_size, row], scratch block tables
+    order, without those that end before position first_keys[b] (a host
+    list; their table entries name some gathered page, whose rows the mask
+    must hide). Returns (rows [pages * block_size, row], scratch block tables
     [B, max pages] int32 numbering the gathered pages consecutively).
     ctx_lens is a host list, so the shapes are known without a device
     read; rows past a sequence's length are whatever the page holds and
@@ -792,9 +805,11 @@ def latent_gather(cache, block_tables, ctx_lens):
     idx, tables, base = [], [], 0
     width = max(max(counts), 1)
     for b, n in enumerate(counts):
-        idx.extend(range(b * mb, b * mb + n))
-        tables.append(list(range(base, base + n)) + [0] * (width - n))
-        base += n
+        skip = min(int(first_keys[b]) // bs, n) if first_keys else 0
+        idx.extend(range(b * mb + skip, b * mb + n))
+        tables.append([0] * skip + list(range(base, base + n - skip))
+                      + [0] * (width - n))
+        base += n - skip
     dev = cache.device
     pages = block_tables.reshape(-1)[
         torch.tensor(idx, dtype=torch.long, device=dev)].long()
@@ -954,3 +969,72 @@ def stream_mix_norm(x, y, mix, w_out, w_in, w, eps: float, out_dtype,
         return h
     return torch_ref.stream_mix_norm(x, y, mix, w_out, w_in, w, eps,
                                      out_dtype, write_x)
+
+
+# ---- sandwich-normed stacks (kernel groups "lnorm", "diag" and "mix") --------
+
+def layer_norm_cast(x, w, b, eps: float, out_dtype):
+    """Layer norm of f32 or bf16 rows [T, H] with f32 weight and bias →
+    out_dtype."""
+    if x.is_cuda:
+        out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+        _K.layer_norm_cast(out, x, w, b, eps)
+        return out
+    return torch_ref.layer_norm_cast(x, w, b, eps, out_dtype)
+
+
+def embed_layer_norm(ids, table, scale: float, w, b, eps: float):
+    """Opens a residual stream: x = table[ids]*scale in f32 and its layer
+    norm in the table's dtype. Returns (x [T, H] f32, h [T, H])."""
+    if ids.is_cuda:
+        shape = (ids.numel(), table.size(1))
+        x = torch.empty(shape, dtype=torch.float32, device=ids.device)
+        h = torch.empty(shape, dtype=table.dtype, device=ids.device)
+        _K.embed_layer_norm(x, h, ids, table, scale, w, b, eps)
+        return x, h
+    return torch_ref.embed_layer_norm(ids, table, scale, w, b, eps)
+
+
+def sandwich_norm_residual(x32, y, w, b, w_next, b_next, eps: float,
+                           out_dtype, y2=None):
+    """Residual step with a layer norm on both sides of a sub-layer, on an
+    f32 stream [T, H]: x32 += ln(y + y2)*w + b in place; returns the next
+    sub-layer's input ln(x32)*w_next + b_next in out_dtype (None when
+    w_next is None). y and y2 (optional) are f32 or bf16, each its own;
+    weights and biases f32."""
+    if x32.is_cuda:
+        h = torch.empty(x32.shape, dtype=out_dtype, device=x32.device) \
+            if w_next is not None else x32
+        _K.sandwich_norm_residual(x32, h, y, _none(y2, y), w, b,
+                                  _none(w_next, y), _none(b_next, y), eps)
+        return h if w_next is not None else None
+    return torch_ref.sandwich_norm_residual(x32, y, w, b, w_next, b_next,
+                                            eps, out_dtype, y2)
+
+
+def gla_scan(q, k, v, gate, low, a2, a_bias, tau: float, q_scale: float,
+             norm_w, state, cu_seqlens, state_slots, seq_starts,
+             norm_eps: float):
+    """Gated linear attention with a decay per key channel: q/k [T, H, D],
+    v/gate [T, H, V] (row strides free), low [T, R] f32 (row stride free),
+    a2 [R, H*D] and a_bias [H*D] f32, norm_w [V] f32, state [slots, H, D, V]
+    f32 in place. alpha = sigmoid(low @ a2 + a_bias)^(1/tau), S <-
+    diag(alpha) S + k v^T, o = S^T q * q_scale, RMS-normed over V with
+    norm_w, times silu(gate). Returns [T, H*V]."""
+    if q.is_cuda:
+        T, H, V = v.shape
+        out = torch.empty(T, H * V, dtype=q.dtype, device=q.device)
+        _K.gla_scan(out, q, k, v, gate, low, a2, a_bias, tau, q_scale, norm_w,
+                    state, cu_seqlens, state_slots, seq_starts, norm_eps)
+        return out
+    return torch_ref.gla_scan(q, k, v, gate, low, a2, a_bias, tau, q_scale,
+                              norm_w, state, cu_seqlens, state_slots,
+                              seq_starts, norm_eps)
+
+
+def scaled_softcap(x, scale: float, cap: float):
+    """x f32, in place: cap*tanh(x*scale/cap) (cap <= 0: x*scale)."""
+    if x.is_cuda:
+        _K.scaled_softcap(x, scale, cap)
+        return x
+    return torch_ref.scaled_softcap(x, scale, cap)

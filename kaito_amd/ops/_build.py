@@ -50,10 +50,12 @@ GROUPS: Dict[str, List[str]] = {
     # latent attention over a paged low-rank cache, hashed bigram embedding
     "latent": ["latent_attention.hip"],
     # matrix recurrences with a decay per state row: generalized delta
-    # rule, gated linear attention with a tied write gate
+    # rule, gated linear attention (tied write gate; low-rank decay)
     "diag": ["diag_delta.hip"],
     # hyper-connected residual streams
     "streams": ["streams.hip"],
+    # layer norms around sub-layers on an f32 residual stream
+    "lnorm": ["layer_norm_f32.hip"],
 }
 
 

@@ -9,9 +9,12 @@
 //                     f = lower + (1 - lower) sigmoid(f_pre + f_bias),
 //                     q = silu(q_pre);
 //                     rms(o) over the value size with a shared weight
+//   gla_scan          S <- diag(alpha) S + k v^T,              o = S^T q
+//                     alpha = sigmoid(low A2 + bias)^(1/tau) from a low-rank
+//                     bottleneck, q scaled; rms(o) as above, times silu(gate)
 //
-// Per head the state S is [D, V] f32 in a slot of its sequence. Both are
-// one recurrence,  S <- diag(d) S - b (u^T S) + k v^T  (the second without
+// Per head the state S is [D, V] f32 in a slot of its sequence. All are
+// one recurrence,  S <- diag(d) S - b (u^T S) + k v^T  (the last two without
 // the removal term), run by three launches:
 //   1. prep (token-parallel, one wave per token and head): activations of
 //      the gates, the unit key, and what lets the read-out be taken from
@@ -30,6 +33,7 @@
 // held; slots < 0 are padding and skipped.
 #include "mix_common.h"
 #include <cstdlib>
+#include <type_traits>
 
 namespace kaito {
 
@@ -120,6 +124,68 @@ __global__ __launch_bounds__(64) void hgrn2_prep_kernel(
   }
   rk = wave_reduce_sum(rk);
   if (lane == 0) srk[(int64_t)t * H + h] = rk;
+}
+
+// ln(sigmoid(z)) without overflow on either side
+KAITO_DEV float log_sigmoid_f(float z) {
+  return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+}
+
+// One wave per (TB tokens, head): a row of A2 is loaded once for all of
+// them. scratch rows: rd (= q*alpha), d (= alpha), k; scalar rk = q.k
+template <typename T, int TB>
+__global__ __launch_bounds__(64) void gla_prep_kernel(
+    float* __restrict__ srd, float* __restrict__ sd, float* __restrict__ sk,
+    float* __restrict__ srk,
+    const T* __restrict__ q, const int64_t q_s0, const int64_t q_s1,
+    const T* __restrict__ k, const int64_t k_s0, const int64_t k_s1,
+    const float* __restrict__ low, const int64_t low_s0,
+    const float* __restrict__ a2,                         // [rank, H*D]
+    const float* __restrict__ a_bias, const float inv_tau,
+    const float q_scale, const int rank, const int NT, const int H,
+    const int D, const int DPAD) {
+  const int t0 = blockIdx.x * TB, h = blockIdx.y, lane = threadIdx.x;
+  const int64_t hd = (int64_t)H * D;
+  float rk[TB];
+#pragma unroll
+  for (int u = 0; u < TB; u++) rk[u] = 0.f;
+  for (int i = lane; i < DPAD; i += 64) {
+    const bool in = i < D;
+    float z[TB];
+    if (in) {
+      const float* col = a2 + (int64_t)h * D + i;
+      const float bias = a_bias[(int64_t)h * D + i];
+#pragma unroll
+      for (int u = 0; u < TB; u++) z[u] = bias;
+      for (int r = 0; r < rank; r++) {
+        const float w = col[r * hd];
+#pragma unroll
+        for (int u = 0; u < TB; u++)
+          z[u] += low[(int64_t)min(t0 + u, NT - 1) * low_s0 + r] * w;
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < TB; u++) {
+      const int t = t0 + u;
+      if (t >= NT) break;
+      float rd = 0.f, d = 0.f, kv = 0.f;
+      if (in) {
+        d = expf(log_sigmoid_f(z[u]) * inv_tau);
+        kv = act_ld(k + (int64_t)t * k_s0 + (int64_t)h * k_s1 + i);
+        const float qv =
+            act_ld(q + (int64_t)t * q_s0 + (int64_t)h * q_s1 + i) * q_scale;
+        rd = qv * d;
+        rk[u] += qv * kv;
+      }
+      const int64_t o = ((int64_t)t * H + h) * DPAD + i;
+      srd[o] = rd; sd[o] = d; sk[o] = kv;
+    }
+  }
+#pragma unroll
+  for (int u = 0; u < TB; u++) {
+    const float v = wave_reduce_sum(rk[u]);
+    if (lane == 0 && t0 + u < NT) srk[(int64_t)(t0 + u) * H + h] = v;
+  }
 }
 
 // ---- recurrence ----------------------------------------------------------------
@@ -286,15 +352,15 @@ __global__ __launch_bounds__(64) void diag_recurrence_kernel(
 }
 
 // ---- epilogue ------------------------------------------------------------------
-// one wave per (token, head): o / sqrt(mean(o^2) + eps) * w * sigmoid(gate);
-// w is indexed over all heads (w_stride = V) or shared by them (0)
+// one wave per (token, head): o / sqrt(mean(o^2) + eps) * w * act(gate), act
+// sigmoid or silu; w is indexed over all heads (w_stride = V) or shared by them (0)
 template <typename T>
 __global__ __launch_bounds__(64) void diag_epilogue_kernel(
     T* __restrict__ out,                                   // [T, H*V]
     const float* __restrict__ o,                           // [T, H, V]
     const T* __restrict__ gate, const int64_t g_s0, const int64_t g_s1,
-    const float* __restrict__ w, const int w_stride, const int H, const int V,
-    const float eps) {
+    const bool gate_silu, const float* __restrict__ w, const int w_stride,
+    const int H, const int V, const float eps) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const float* orow = o + ((int64_t)t * H + h) * V;
   float ss = 0.f;
@@ -306,7 +372,10 @@ __global__ __launch_bounds__(64) void diag_epilogue_kernel(
   T* dst = out + ((int64_t)t * H + h) * V;
   for (int i = lane; i < V; i += 64) {
     float y = orow[i] * inv * wr[i];
-    if (gr) y *= sigmoid_f(act_ld(gr + i));
+    if (gr) {
+      const float g = act_ld(gr + i);
+      y *= gate_silu ? silu_f(g) : sigmoid_f(g);
+    }
     act_st(dst + i, y);
   }
 }
@@ -429,7 +498,7 @@ void diag_delta_rule(at::Tensor out, at::Tensor r, at::Tensor k, at::Tensor v,
         state.data_ptr<float>(), c);
     hipLaunchKernelGGL((diag_epilogue_kernel<act_t>), dim3(T, H), dim3(64),
         0, stream, (act_t*)out.data_ptr(), o.data_ptr<float>(),
-        (const act_t*)gate.data_ptr(), gate.stride(0), gate.stride(1),
+        (const act_t*)gate.data_ptr(), gate.stride(0), gate.stride(1), false,
         norm_w.data_ptr<float>(), D, H, D, (float)norm_eps);
   });
 }
@@ -480,7 +549,70 @@ void hgrn2_scan(at::Tensor out, at::Tensor q, at::Tensor v, at::Tensor f_pre,
         state.data_ptr<float>(), c);
     hipLaunchKernelGGL((diag_epilogue_kernel<act_t>), dim3(T, H), dim3(64),
         0, stream, (act_t*)out.data_ptr(), o.data_ptr<float>(),
-        (const act_t*)nullptr, (int64_t)0, (int64_t)0,
+        (const act_t*)nullptr, (int64_t)0, (int64_t)0, false,
+        norm_w.data_ptr<float>(), 0, H, V, (float)norm_eps);
+  });
+}
+
+void gla_scan(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v,
+              at::Tensor gate, at::Tensor low, at::Tensor a2,
+              at::Tensor a_bias, double tau, double q_scale,
+              at::Tensor norm_w, at::Tensor state, at::Tensor cu_seqlens,
+              at::Tensor state_slots, at::Tensor seq_starts,
+              double norm_eps) {
+  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && is_act_dtype(q) &&
+              v.dim() == 3);
+  const int T = q.size(0), H = q.size(1), D = q.size(2), V = v.size(2);
+  TORCH_CHECK(D >= 1 && D <= 256, "state rows per head: 1..256, got ", D);
+  check_heads(q, T, H, D, "q"); check_heads(k, T, H, D, "k");
+  check_heads(v, T, H, V, "v"); check_heads(gate, T, H, V, "gate");
+  TORCH_CHECK(k.dtype() == q.dtype() && v.dtype() == q.dtype() &&
+              gate.dtype() == q.dtype());
+  TORCH_CHECK(low.is_cuda() && low.dtype() == at::kFloat && low.dim() == 2 &&
+              low.size(0) == T && low.stride(1) == 1,
+              "decay bottleneck: f32 [T, rank]");
+  const int rank = low.size(1);
+  KAITO_CHECK_F32(a2); KAITO_CHECK_F32(a_bias);
+  TORCH_CHECK(a2.dim() == 2 && a2.size(0) == rank && a2.size(1) == H * D &&
+              a_bias.numel() == H * D && tau > 0);
+  KAITO_CHECK_F32(norm_w); KAITO_CHECK_F32(state);
+  TORCH_CHECK(norm_w.numel() == V);
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D &&
+              state.size(3) == V);
+  TORCH_CHECK(out.is_contiguous() && out.dtype() == q.dtype() &&
+              out.dim() == 2 && out.size(0) == T && out.size(1) == H * V);
+  const ChunkArgs c = check_chunks(cu_seqlens, state_slots, seq_starts, T);
+  if (T == 0) return;
+  auto stream = at::hip::getCurrentHIPStream();
+  const int DPAD = padded_rows(D);
+  auto f32 = q.options().dtype(at::kFloat);
+  at::Tensor vec = at::empty({3, T, H, DPAD}, f32);
+  at::Tensor sca = at::empty({T, H}, f32);
+  at::Tensor o = at::empty({T, H, V}, f32);
+  float* vp = vec.data_ptr<float>();
+  const int64_t vs = (int64_t)T * H * DPAD;
+  float* srd = vp, *sd = vp + vs, *sk = vp + 2 * vs;
+  float* srk = sca.data_ptr<float>();
+  KAITO_DISPATCH_ACT(q, {
+    auto prep = [&](auto tb) {
+      constexpr int TB = decltype(tb)::value;
+      hipLaunchKernelGGL((gla_prep_kernel<act_t, TB>),
+          dim3((T + TB - 1) / TB, H), dim3(64), 0, stream, srd, sd, sk, srk,
+          (const act_t*)q.data_ptr(), q.stride(0), q.stride(1),
+          (const act_t*)k.data_ptr(), k.stride(0), k.stride(1),
+          low.data_ptr<float>(), low.stride(0), a2.data_ptr<float>(),
+          a_bias.data_ptr<float>(), (float)(1.0 / tau), (float)q_scale, rank,
+          T, H, D, DPAD);
+    };
+    if ((int64_t)T * H >= 16384) prep(std::integral_constant<int, 8>{});
+    else prep(std::integral_constant<int, 1>{});
+    launch_recurrence<act_t, false>(stream, c.B, H, D, V,
+        o.data_ptr<float>(), nullptr, srd, sd, nullptr, sk, nullptr, srk,
+        (const act_t*)v.data_ptr(), v.stride(0), v.stride(1),
+        state.data_ptr<float>(), c);
+    hipLaunchKernelGGL((diag_epilogue_kernel<act_t>), dim3(T, H), dim3(64),
+        0, stream, (act_t*)out.data_ptr(), o.data_ptr<float>(),
+        (const act_t*)gate.data_ptr(), gate.stride(0), gate.stride(1), true,
         norm_w.data_ptr<float>(), 0, H, V, (float)norm_eps);
   });
 }
@@ -490,8 +622,10 @@ void hgrn2_scan(at::Tensor out, at::Tensor q, at::Tensor v, at::Tensor f_pre,
 TORCH_LIBRARY_FRAGMENT(kaito, m) {
   m.def("diag_delta_rule(Tensor(a!) out, Tensor r, Tensor k, Tensor v, Tensor w_pre, Tensor a_pre, Tensor a_bias, Tensor gate, Tensor norm_w, Tensor(b!) state, Tensor cu_seqlens, Tensor state_slots, Tensor seq_starts, float decay_rate, float k_eps, float norm_eps) -> ()");
   m.def("hgrn2_scan(Tensor(a!) out, Tensor q, Tensor v, Tensor f_pre, Tensor f_bias, Tensor lower, Tensor norm_w, Tensor(b!) state, Tensor cu_seqlens, Tensor state_slots, Tensor seq_starts, float norm_eps) -> ()");
+  m.def("gla_scan(Tensor(a!) out, Tensor q, Tensor k, Tensor v, Tensor gate, Tensor low, Tensor a2, Tensor a_bias, float tau, float q_scale, Tensor norm_w, Tensor(b!) state, Tensor cu_seqlens, Tensor state_slots, Tensor seq_starts, float norm_eps) -> ()");
 }
 TORCH_LIBRARY_IMPL(kaito, CUDA, m) {
   m.impl("diag_delta_rule", &kaito::diag_delta_rule);
   m.impl("hgrn2_scan", &kaito::hgrn2_scan);
+  m.impl("gla_scan", &kaito::gla_scan);
 }

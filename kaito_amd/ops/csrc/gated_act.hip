@@ -8,6 +8,7 @@
 //   gelu_glu:     [gate | up] rows [T, 2F] -> gelu_tanh(gate) * up
 //   relu_glu:     [gate | up] rows [T, 2F] -> relu(gate) * up
 //   relu2:        relu(x)^2
+//   scaled_softcap: cap * tanh(x * scale / cap), f32 in place (logits)
 #include "mix_common.h"
 
 namespace kaito {
@@ -113,7 +114,41 @@ __global__ void unary_glu_vec_kernel(T* __restrict__ out,
       *reinterpret_cast<const float4_t*>(ov);
 }
 
+// V elements per thread
+template <int V>
+__global__ void scaled_softcap_kernel(float* __restrict__ x, const int64_t n,
+                                      const float scale, const float cap) {
+  const int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * V;
+  if (i >= n) return;
+  float v[V];
+#pragma unroll
+  for (int e = 0; e < V; e++) v[e] = x[i + e] * scale;
+  if (cap > 0.f) {
+#pragma unroll
+    for (int e = 0; e < V; e++) v[e] = cap * tanhf(v[e] / cap);
+  }
+#pragma unroll
+  for (int e = 0; e < V; e++) x[i + e] = v[e];
+}
+
 }  // namespace
+
+void scaled_softcap(at::Tensor x, double scale, double cap) {
+  KAITO_CHECK_F32(x);
+  const int64_t n = x.numel();
+  if (n == 0) return;
+  auto stream = at::hip::getCurrentHIPStream();
+  const bool vec = n % 4 == 0 && (uintptr_t)x.data_ptr() % 16 == 0;
+  const int64_t threads = vec ? n / 4 : n;
+  TORCH_CHECK((threads + 255) / 256 < (1ll << 31));
+  const dim3 grid((unsigned)((threads + 255) / 256));
+  if (vec)
+    hipLaunchKernelGGL(scaled_softcap_kernel<4>, grid, dim3(256), 0, stream,
+        x.data_ptr<float>(), n, (float)scale, (float)cap);
+  else
+    hipLaunchKernelGGL(scaled_softcap_kernel<1>, grid, dim3(256), 0, stream,
+        x.data_ptr<float>(), n, (float)scale, (float)cap);
+}
 
 void clamped_glu(at::Tensor out, at::Tensor gu, double limit, double alpha) {
   TORCH_CHECK(gu.is_cuda() && gu.dim() == 2 && gu.stride(1) == 1 &&
@@ -231,6 +266,7 @@ TORCH_LIBRARY_FRAGMENT(kaito, m) {
   m.def("gelu_glu(Tensor(a!) out, Tensor gu) -> ()");
   m.def("relu_glu(Tensor(a!) out, Tensor gu) -> ()");
   m.def("relu2(Tensor(a!) out, Tensor x) -> ()");
+  m.def("scaled_softcap(Tensor(a!) x, float scale, float cap) -> ()");
 }
 TORCH_LIBRARY_IMPL(kaito, CUDA, m) {
   m.impl("clamped_glu", &kaito::clamped_glu);
@@ -238,4 +274,5 @@ TORCH_LIBRARY_IMPL(kaito, CUDA, m) {
   m.impl("gelu_glu", &kaito::gelu_glu);
   m.impl("relu_glu", &kaito::relu_glu);
   m.impl("relu2", &kaito::relu2);
+  m.impl("scaled_softcap", &kaito::scaled_softcap);
 }

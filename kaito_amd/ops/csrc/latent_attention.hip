@@ -9,6 +9,7 @@
 // space: with q_c = W_uk,h^T q_h,
 //
 //   score(i, j) = (q_c,i . c_j + q_rot,i . k_rot,j) * scale,   j <= i
+//                 (with a window only i - j < window)
 //   out_c,i     = sum_j softmax_j(score)(+ sink) * c_j
 //
 // and W_uv,h is applied to out_c afterwards. One pass over the cache rows
@@ -175,7 +176,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
     const int* __restrict__ block_tables, const int max_blocks,
     const int* __restrict__ token_seq, const int64_t* __restrict__ positions,
     const float scale, const float* __restrict__ sinks, const int H,
-    const int DT, const int rank, const int BS) {
+    const int DT, const int rank, const int BS, const int window) {
   extern __shared__ __align__(16) unsigned char lds_raw[];
   const int RS = DT + lds_pad<T>::v;                 // padded row, elements
   float* q_s = reinterpret_cast<float*>(lds_raw);   // [HT][DT]
@@ -192,6 +193,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
     return;
   }
   const int nkeys = (int)positions[t] + 1;
+  const int first = window > 0 ? max(0, nkeys - window) : 0;
   const int* bt = block_tables + (int64_t)b * max_blocks;
 
   for (int i = tid; i < LA_HT * DT; i += 256) {
@@ -205,7 +207,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
   float m_run = sink ? sinks[h] : -INFINITY, l_run = sink ? 1.0f : 0.f;
   const int wave = tid >> 6, lane = tid & 63;
 
-  for (int k0 = 0; k0 < nkeys; k0 += LA_KT) {
+  for (int k0 = first; k0 < nkeys; k0 += LA_KT) {
     const int nk = min(LA_KT, nkeys - k0);
     __syncthreads();              // q_s ready / previous tile consumed
     for (int r = wave; r < nk; r += 4) {
@@ -287,7 +289,8 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(
     const int* __restrict__ block_tables, const int max_blocks,
     const int* __restrict__ token_seq, const int64_t* __restrict__ positions,
     const float scale, const float* __restrict__ sinks, const int H,
-    const int DT, const int rank, const int BS, const int S) {
+    const int DT, const int rank, const int BS, const int S,
+    const int window) {
   extern __shared__ __align__(16) unsigned char lds_raw[];
   const int DTp = (DT + 31) & ~31, RS = DTp + 8;
   const int rankp = (rank + 15) & ~15;
@@ -306,9 +309,13 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(
   const int sh = tid >> 4, sj = tid & 15;       // softmax role: head, key pair
   const int b = token_seq[t];
   const int nkeys = b < 0 ? 0 : (int)positions[t] + 1;
-  const int nt_all = (nkeys + 31) >> 5;
-  const int tile_lo = (int)((int64_t)nt_all * split / S);
-  const int tile_hi = (int)((int64_t)nt_all * (split + 1) / S);
+  // visible keys first .. nkeys - 1; every 32-row tile from t_first on
+  // holds at least one of them
+  const int first = window > 0 ? max(0, nkeys - window) : 0;
+  const int t_first = first >> 5;
+  const int nt_all = ((nkeys + 31) >> 5) - t_first;
+  const int tile_lo = t_first + (int)((int64_t)nt_all * split / S);
+  const int tile_hi = t_first + (int)((int64_t)nt_all * (split + 1) / S);
   const int* bt = block_tables + (int64_t)max(b, 0) * max_blocks;
 
   // zero what staging never writes: the k padding of the rows and the
@@ -362,7 +369,7 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(
 
   for (int tile = tile_lo; tile < tile_hi; tile++) {
     const int k0 = tile << 5;
-    const int nk = min(32, nkeys - k0);
+    const int nk = min(32, nkeys - k0), nf = first - k0;   // first visible
     __syncthreads();            // previous tile consumed
 #pragma unroll
     for (int i = 0; i < MAXC; i++) {
@@ -416,12 +423,14 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(
         s0 += part_s[(w * 16 + sh) * 32 + sj];
         s1 += part_s[(w * 16 + sh) * 32 + sj + 16];
       }
-      s0 = sj < nk ? s0 * scale : -INFINITY;
-      s1 = sj + 16 < nk ? s1 * scale : -INFINITY;
+      const bool v0 = sj < nk && sj >= nf;
+      const bool v1 = sj + 16 < nk && sj + 16 >= nf;
+      s0 = v0 ? s0 * scale : -INFINITY;
+      s1 = v1 ? s1 * scale : -INFINITY;
       const float m_new =
           fmaxf(m_run, group_reduce_max<16>(fmaxf(s0, s1)));
-      const float p0 = sj < nk ? expf(s0 - m_new) : 0.f;
-      const float p1 = sj + 16 < nk ? expf(s1 - m_new) : 0.f;
+      const float p0 = v0 ? expf(s0 - m_new) : 0.f;
+      const float p1 = v1 ? expf(s1 - m_new) : 0.f;
       const float ps = group_reduce_sum<16>(p0 + p1);
       const float corr = expf(m_run - m_new);
       l_run = l_run * corr + ps;
@@ -651,7 +660,8 @@ void latent_rope_cache_write(at::Tensor q_out, at::Tensor q, at::Tensor dkv,
 
 void latent_attention(at::Tensor out, at::Tensor q, at::Tensor cache,
                       at::Tensor block_tables, at::Tensor token_seq,
-                      at::Tensor positions, double scale, at::Tensor sinks) {
+                      at::Tensor positions, double scale, at::Tensor sinks,
+                      int64_t window) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() &&
               is_act_dtype(q));
   const int T = q.size(0), H = q.size(1), DT = q.size(2);
@@ -670,6 +680,7 @@ void latent_attention(at::Tensor out, at::Tensor q, at::Tensor cache,
   const bool sk = sinks.numel() > 0;
   if (sk) { KAITO_CHECK_F32(sinks); TORCH_CHECK(sinks.numel() == H); }
   TORCH_CHECK((int64_t)cache.size(0) * BS < (1ll << 31));
+  TORCH_CHECK(window >= 0 && window < (1 << 30));
   if (T == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
   // bf16 with 16-byte chunks per row: the MFMA kernel
@@ -680,6 +691,8 @@ void latent_attention(at::Tensor out, at::Tensor q, at::Tensor cache,
     // (one workgroup per CU: a tile pair of 32 rows takes most of its LDS)
     int S = (256 + T * tiles_h - 1) / std::max(1, T * tiles_h);
     S = std::max(1, std::min(S, 16));
+    // a window spans few tiles: no more splits than that
+    if (window > 0) S = std::min(S, (int)((window + 62) / 32));
     const int DTp = (DT + 31) & ~31, rankp = (rank + 15) & ~15;
     const size_t lds = (size_t)(32 * (DTp + 8) + rankp * LM_KTP +
                                 2 * 16 * LM_KTP) * 2 +
@@ -705,7 +718,7 @@ void latent_attention(at::Tensor out, at::Tensor q, at::Tensor cache,
           block_tables.data_ptr<int>(), (int)block_tables.size(1),
           token_seq.data_ptr<int>(), positions.data_ptr<int64_t>(),
           (float)scale, sk ? sinks.data_ptr<float>() : nullptr, H, DT, rank,
-          BS, S);
+          BS, S, (int)window);
     };
     if (small) launch(&latent_attention_mfma_kernel<2, 2>);
     else launch(&latent_attention_mfma_kernel<5, 8>);
@@ -735,7 +748,8 @@ void latent_attention(at::Tensor out, at::Tensor q, at::Tensor cache,
         (const act_t*)cache.data_ptr(), block_tables.data_ptr<int>(),
         (int)block_tables.size(1), token_seq.data_ptr<int>(),
         positions.data_ptr<int64_t>(), (float)scale,
-        sk ? sinks.data_ptr<float>() : nullptr, H, DT, rank, BS);
+        sk ? sinks.data_ptr<float>() : nullptr, H, DT, rank, BS,
+        (int)window);
   });
 }
 
@@ -774,7 +788,7 @@ void latent_expand(at::Tensor k_s, at::Tensor v_s, at::Tensor kn,
 TORCH_LIBRARY_FRAGMENT(kaito, m) {
   m.def("bigram_embed(Tensor(a!) out, Tensor ids, Tensor embed, float scale, Tensor table, int buckets, int mul_prev, int mul_cur, Tensor(b!) prev_state, Tensor cu_seqlens, Tensor state_slots, Tensor seq_starts, Tensor token_seq) -> ()");
   m.def("latent_rope_cache_write(Tensor(a!) q_out, Tensor q, Tensor dkv, Tensor norm_w, float eps, Tensor(b!) cache, Tensor slot_mapping, Tensor positions, Tensor inv_freq, int dim, bool interleaved, float rot_mag) -> ()");
-  m.def("latent_attention(Tensor(a!) out, Tensor q, Tensor cache, Tensor block_tables, Tensor token_seq, Tensor positions, float scale, Tensor sinks) -> ()");
+  m.def("latent_attention(Tensor(a!) out, Tensor q, Tensor cache, Tensor block_tables, Tensor token_seq, Tensor positions, float scale, Tensor sinks, int window) -> ()");
   m.def("latent_expand(Tensor(a!) k_s, Tensor(b!) v_s, Tensor kn, Tensor vv, Tensor lat, int H, int D, int V, int rank) -> ()");
 }
 TORCH_LIBRARY_IMPL(kaito, CUDA, m) {

@@ -1,7 +1,7 @@
 // Expert choice for routed feed-forwards, in two launches.
 //
 //   moe_route: one wave per token. s = softmax(logits); choice = s +
-//     correction; the outputs form `groups` equal groups of neighbours, a
+//     correction (none given: s); the outputs form `groups` equal groups of neighbours, a
 //     group scores its largest choice, only the `keep` best groups stay
 //     eligible; the `top` largest eligible choices are taken (ties: lower
 //     index). Weights are the taken s (without the correction), divided by
@@ -61,7 +61,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
   for (int r = 0; r < NPL; r++) {
     const int e = r * 64 + lane;
     s[r] = s[r] / sum;
-    ch[r] = e < N ? s[r] + correction[e] : -INFINITY;
+    ch[r] = e < N ? s[r] + (correction ? correction[e] : 0.f) : -INFINITY;
   }
   if (groups > 1) {
     const int n = N / groups;
@@ -155,12 +155,14 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(
 void moe_route(at::Tensor topi, at::Tensor topw, at::Tensor w_id,
                at::Tensor logits, at::Tensor correction, int64_t n_real,
                int64_t groups, int64_t keep, bool renorm, double scale) {
-  KAITO_CHECK_F32(logits); KAITO_CHECK_F32(correction);
+  KAITO_CHECK_F32(logits);
+  const bool corr = correction.numel() > 0;
+  if (corr) KAITO_CHECK_F32(correction);
   KAITO_CHECK_I32(topi); KAITO_CHECK_F32(topw); KAITO_CHECK_F32(w_id);
   TORCH_CHECK(logits.dim() == 2 && topi.dim() == 2);
   const int T = logits.size(0), N = logits.size(1), top = topi.size(1);
   TORCH_CHECK(topi.size(0) == T && topw.sizes() == topi.sizes() &&
-              w_id.numel() == T && correction.numel() == N);
+              w_id.numel() == T && (!corr || correction.numel() == N));
   TORCH_CHECK(N >= 1 && N <= ROUTE_MAX && top >= 1 && top <= 64 && top <= N);
   TORCH_CHECK(groups >= 1 && groups <= 64 && N % groups == 0 && keep >= 1 &&
               keep <= groups);
@@ -170,7 +172,8 @@ void moe_route(at::Tensor topi, at::Tensor topw, at::Tensor w_id,
     hipLaunchKernelGGL((moe_route_kernel<decltype(npl)::value>),
         dim3((T + 3) / 4), dim3(256), 0, stream, topi.data_ptr<int>(),
         topw.data_ptr<float>(), w_id.data_ptr<float>(),
-        logits.data_ptr<float>(), correction.data_ptr<float>(), T, N,
+        logits.data_ptr<float>(),
+        corr ? correction.data_ptr<float>() : nullptr, T, N,
         (int)n_real, top, (int)groups, (int)keep, renorm, (float)scale);
   };
   if (N <= 64) launch(std::integral_constant<int, 1>{});

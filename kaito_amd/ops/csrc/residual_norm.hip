@@ -6,7 +6,8 @@
 //       m = (rms(y) * w_y + rms(y2) * w_y2) / 2        (two side by side)
 //     and x32's rounding to the activation dtype is emitted for the next
 //     sub-layer in the same pass.
-//   rms_norm_cast: rms(x) * w for f32 or bf16 rows → f32 or bf16.
+//   rms_norm_cast: rms(x) * w for f32 or bf16 rows (row stride free) → f32
+//   or bf16.
 //
 // and for pre-norm models with an f32 stream:
 //
@@ -72,11 +73,11 @@ __global__ void post_norm_residual_kernel(
 
 template <typename TI, typename TO>
 __global__ void rms_norm_cast_kernel(
-    TO* __restrict__ out, const TI* __restrict__ x,
+    TO* __restrict__ out, const TI* __restrict__ x, const int64_t x_s0,
     const float* __restrict__ w, const int H, const float eps) {
   __shared__ float red[16];
   const int row = blockIdx.x;
-  const TI* xr = x + (int64_t)row * H;
+  const TI* xr = x + (int64_t)row * x_s0;
   float ss = 0.f;
   for (int i = threadIdx.x; i < H; i += blockDim.x) {
     const float v = act_ld(xr + i);
@@ -274,9 +275,10 @@ void residual_add_norm(at::Tensor x32, at::Tensor h_out, at::Tensor y,
 }
 
 void rms_norm_cast(at::Tensor out, at::Tensor x, at::Tensor w, double eps) {
-  TORCH_CHECK(x.is_cuda() && x.is_contiguous() && is_act_dtype(x) &&
+  TORCH_CHECK(x.is_cuda() && is_act_dtype(x) && x.dim() >= 1 &&
+              (x.is_contiguous() || (x.dim() == 2 && x.stride(1) == 1)) &&
               out.is_contiguous() && is_act_dtype(out) &&
-              out.sizes() == x.sizes() && x.dim() >= 1);
+              out.sizes() == x.sizes());
   const int H = x.size(-1);
   const int T = H > 0 ? x.numel() / H : 0;
   KAITO_CHECK_F32(w);
@@ -289,7 +291,9 @@ void rms_norm_cast(at::Tensor out, at::Tensor x, at::Tensor w, double eps) {
     KAITO_DISPATCH_ACT(out, {
       hipLaunchKernelGGL((rms_norm_cast_kernel<in_t, act_t>), dim3(T),
           dim3(threads), 0, stream, (act_t*)out.data_ptr(),
-          (const in_t*)x.data_ptr(), w.data_ptr<float>(), H, (float)eps);
+          (const in_t*)x.data_ptr(),
+          x.is_contiguous() ? (int64_t)H : x.stride(0), w.data_ptr<float>(),
+          H, (float)eps);
     });
   });
 }

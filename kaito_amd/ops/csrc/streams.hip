@@ -22,23 +22,6 @@ namespace kaito {
 
 namespace {
 
-KAITO_DEV float4_t act_ld4(const float* p) {
-  return *reinterpret_cast<const float4_t*>(p);
-}
-KAITO_DEV float4_t act_ld4(const bf16_act* p) {
-  const short4_t r = *reinterpret_cast<const short4_t*>(p);
-  return float4_t{bf16_to_f32(r[0]), bf16_to_f32(r[1]), bf16_to_f32(r[2]),
-                  bf16_to_f32(r[3])};
-}
-KAITO_DEV void act_st4(float* p, const float4_t v) {
-  *reinterpret_cast<float4_t*>(p) = v;
-}
-KAITO_DEV void act_st4(bf16_act* p, const float4_t v) {
-  *reinterpret_cast<short4_t*>(p) =
-      short4_t{f32_to_bf16(v[0]), f32_to_bf16(v[1]), f32_to_bf16(v[2]),
-               f32_to_bf16(v[3])};
-}
-
 template <int S, int NV, typename T, typename TO>
 __global__ __launch_bounds__(512) void stream_mix_norm_kernel(
     float* __restrict__ x, TO* __restrict__ h_out, const T* __restrict__ y,

@@ -4,6 +4,9 @@
 //
 //   score(i, j) = cap * tanh(q_i . k_j * scale / cap)      (cap > 0)
 //                 - r1_h * ln(1 + r2_h * (i - j))           (r1 given)
+//                 + db_h[min(i - j, N - 1)]               (table given)
+//                 (the product also times 1 + c * ln(floor((i + 1) / every)
+//                 + 1), a query temperature, when c != 0)
 //   visible:      j <= i and (i - j < window or j < keep_first)
 //                 (window <= 0: every j <= i); or, with chunk > 0,
 //                 j <= i and floor(j / chunk) == floor(i / chunk) on
@@ -248,6 +251,11 @@ __global__ __launch_bounds__(256) void qk_norm_cache_write_vec_kernel(
 }
 
 // ---- attention ------------------------------------------------------------
+KAITO_DEV float query_temp(const int pos, const float coef, const int every) {
+  return coef != 0.f
+      ? 1.0f + coef * logf((float)((pos + 1) / every + 1)) : 1.0f;
+}
+
 template <typename T>
 KAITO_DEV float dot_row(const float* __restrict__ q, const T* __restrict__ k,
                         const int D);
@@ -297,7 +305,8 @@ __global__ void window_attention_kernel(
     const int D, const int V, const int BS, const int keep_first,
     const float* __restrict__ sinks, const int chunk,
     const float* __restrict__ pb, const T* __restrict__ gate,
-    const int64_t gate_s0) {
+    const int64_t gate_s0, const float* __restrict__ db, const int db_n,
+    const float temp_coef, const int temp_every) {
   extern __shared__ float lds[];
   const int KT = blockDim.x;            // keys per tile
   float* q_s = lds;                     // [D]
@@ -322,6 +331,7 @@ __global__ void window_attention_kernel(
   const int* bt = block_tables + (int64_t)b * max_blocks;
   const float hr1 = r1 ? r1[h] : 0.0f, hr2 = r1 ? r2[h] : 0.0f;
 
+  const float sc = scale * query_temp(pos, temp_coef, temp_every);
   for (int d = tid; d < D; d += KT)
     q_s[d] = act_ld(q + ((int64_t)t * H + h) * D + d);
 
@@ -344,9 +354,10 @@ __global__ void window_attention_kernel(
       const int page = bt[j / BS];
       const int64_t rowi = ((int64_t)page * G + g) * BS + (j % BS);
       blk_s[tid] = (int)rowi;
-      s = dot_row<T>(q_s, k_cache + rowi * D, D) * scale;
+      s = dot_row<T>(q_s, k_cache + rowi * D, D) * sc;
       if (softcap > 0.f) s = softcap * tanhf(s / softcap);
       if (r1) s -= hr1 * log1pf(hr2 * (float)(pos - j));
+      if (db) s += db[(int64_t)h * db_n + min(pos - j, db_n - 1)];
     }
     float corr = 1.0f;
     if (pb) {
@@ -409,7 +420,8 @@ constexpr int WQ_TILE = 64;
 constexpr int WKV_TILE = 32;
 constexpr int WPAD = 40;
 
-template <int D, int DV, bool SIG>
+// DB: distance-bias table and query temperature (a softmax variant)
+template <int D, int DV, bool SIG, bool DB>
 __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
     short* __restrict__ out,              // [T, H, DV]
     const short* __restrict__ q,          // [T, H, D]
@@ -422,7 +434,9 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
     const float* __restrict__ r2, const int window, const int H, const int G,
     const int BS, const int keep_first, const float* __restrict__ sinks,
     const int chunk, const float* __restrict__ pb,
-    const short* __restrict__ gate, const int64_t gate_s0) {
+    const short* __restrict__ gate, const int64_t gate_s0,
+    const float* __restrict__ db, const int db_n, const float temp_coef,
+    const int temp_every) {
   constexpr int KK = D / 32;
   constexpr int DT = DV / 16;
   const int tile = blockIdx.x;
@@ -450,6 +464,8 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   // tile keep ~16 mantissa bits of the f32 weight in the P.V product
   __shared__ short lds_p[4][16 * WPAD];
   __shared__ short lds_pl[4][16 * WPAD];
+  // the tile's bias by q row - key + WKV_TILE - 1
+  __shared__ float lds_db[DB ? WQ_TILE + WKV_TILE : 1];
 
   const int qrow = q0 + wave * 16 + lo;
   const int qtok = tok0 + (qrow < q_len ? qrow : q_len - 1);
@@ -459,7 +475,11 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
     qfrag[kk] = *reinterpret_cast<const bf16x8*>(
         q + ((int64_t)qtok * H + h) * D + kk * 32 + hi * 8);
 
-  float mrow[4], lrow[4];
+  float mrow[4], lrow[4], qsc[4];
+#pragma unroll
+  for (int r = 0; r < 4; r++)
+    qsc[r] = DB ? scale * query_temp(q_abs0 + q0 + wave * 16 + hi * 4 + r,
+                                     temp_coef, temp_every) : scale;
   f32x4 ofrag[DT];
 #pragma unroll
   for (int r = 0; r < 4; r++) {
@@ -500,6 +520,11 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
 #pragma unroll
       for (int j = 0; j < 8; j++) lds_vt[(col + j) * WPAD + row] = vd[j];
     }
+    if (DB && threadIdx.x < WQ_TILE + WKV_TILE - 1) {
+      const int dist = q_abs0 + q0 - kv0 + (int)threadIdx.x - (WKV_TILE - 1);
+      lds_db[threadIdx.x] =
+          db[(int64_t)h * db_n + min(max(dist, 0), db_n - 1)];
+    }
     __syncthreads();
 
     f32x4 sfrag[2];
@@ -525,11 +550,13 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
         const int qr = q0 + wave * 16 + hi * 4 + r;
         const int q_abs = q_abs0 + qr;
         const int kvp = kv0 + kt * 16 + lo;
-        float sv = sfrag[kt][r] * scale;
+        float sv = sfrag[kt][r] * (DB ? qsc[r] : scale);
         if (softcap > 0.f)          // cap * tanh(s / cap), via exp
           sv = softcap * (1.0f - 2.0f / (__expf(2.0f * sv * inv_cap) + 1.0f));
         const int dist = q_abs - kvp;
         if (r1) sv -= hr1 * __logf(1.0f + hr2 * (float)max(dist, 0));
+        if (DB) sv += lds_db[wave * 16 + hi * 4 + r - kt * 16 - lo +
+                             WKV_TILE - 1];
         if (dist < 0 || kvp >= kv_len || qr >= q_len ||
             (window > 0 && dist >= window && kvp >= keep_first) ||
             (chunk > 0 && kvp < (q_abs / chunk) * chunk)) sv = -1e30f;
@@ -629,7 +656,8 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
     const int D, const int V, const int BS, const int KT,
     const int keep_first, const float* __restrict__ sinks, const int chunk,
     const float* __restrict__ pb, const T* __restrict__ gate,
-    const int64_t gate_s0) {
+    const int64_t gate_s0, const float* __restrict__ db, const int db_n,
+    const float temp_coef, const int temp_every) {
   constexpr int VEC = 16 / (int)sizeof(T);
   extern __shared__ float lds[];
   float* s_s = lds;                            // [RT][KT]
@@ -660,6 +688,7 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
   const int nkeys = nfirst + pos - lo + 1;
   const int* bt = block_tables + (int64_t)b * max_blocks;
   const int nchunks = D / VEC;
+  const float sc = scale * query_temp(pos, temp_coef, temp_every);
 
   float qreg[RT][NCH][VEC];
 #pragma unroll
@@ -745,7 +774,7 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
           for (int i = 0; i < NCH; i++)
 #pragma unroll
             for (int e = 0; e < VEC; e++) dot += qreg[r][i][e] * kv[un][i][e];
-          float sv = group_reduce_sum<8>(dot) * scale;
+          float sv = group_reduce_sum<8>(dot) * sc;
           if (softcap > 0.f) sv = softcap * tanhf(sv / softcap);
           if (r1) sv -= hr1[r] * log1pf(hr2[r] * dist);
           if (pb) sv = sigmoid_f(sv + hpb[r]);
@@ -759,6 +788,14 @@ __global__ __launch_bounds__(256) void window_attention_decode_kernel(
     // (sigmoid weights have none: l and c stay 1)
     for (int r = pb ? nr : wave; r < nr; r += 4) {
       float mx = -INFINITY;
+      if (db) {                      // the bias joins here, lanes over keys
+        const float* dr = db + (int64_t)(h0 + r) * db_n;
+        for (int kk = lane; kk < nk; kk += 64) {
+          const int kx = k0 + kk;
+          const int dist = pos - (kx < nfirst ? kx : lo + (kx - nfirst));
+          s_s[r * KT + kk] += dr[min(dist, db_n - 1)];
+        }
+      }
       for (int kk = lane; kk < nk; kk += 64) mx = fmaxf(mx, s_s[r * KT + kk]);
       mx = wave_reduce_max(mx);
       const float m_old = m_s[r];
@@ -847,7 +884,8 @@ void launch_decode(int nch, dim3 grid, size_t lds_bytes, hipStream_t stream,
                    const float* r2, int window, int H, int G, int D, int V,
                    int BS, int KT, int keep_first, const float* sinks,
                    int chunk, const float* pb, const T* gate,
-                   int64_t gate_s0) {
+                   int64_t gate_s0, const float* db, int db_n,
+                   float temp_coef, int temp_every) {
 #define KAITO_WDEC(NCH_)                                                     \
   if (nch == NCH_) {                                                         \
     hipLaunchKernelGGL((window_attention_decode_kernel<T, RT, NCH_>), grid,  \
@@ -856,7 +894,8 @@ void launch_decode(int nch, dim3 grid, size_t lds_bytes, hipStream_t stream,
         (const T*)v_cache.data_ptr(), block_tables.data_ptr<int>(),          \
         (int)block_tables.size(1), token_seq.data_ptr<int>(),                \
         positions.data_ptr<int64_t>(), scale, softcap, r1, r2, window, H, G, \
-        D, V, BS, KT, keep_first, sinks, chunk, pb, gate, gate_s0);          \
+        D, V, BS, KT, keep_first, sinks, chunk, pb, gate, gate_s0, db, db_n, \
+        temp_coef, temp_every);                                              \
     return;                                                                  \
   }
   KAITO_WDEC(1) KAITO_WDEC(2) KAITO_WDEC(4)
@@ -882,6 +921,20 @@ void check_weights_and_gate(const at::Tensor& q, const at::Tensor& sinks,
     TORCH_CHECK(gate.is_cuda() && gate.dim() == 2 && gate.stride(1) == 1 &&
                 gate.dtype() == q.dtype() && gate.size(0) == q.size(0) &&
                 gate.size(1) == q.size(1));
+}
+
+// Table entries per head (0 = no distance bias).
+int check_distance_bias(const at::Tensor& q, const at::Tensor& dist_bias,
+                        const at::Tensor& sig_bias, double temp_coef,
+                        int64_t temp_every) {
+  TORCH_CHECK(temp_every >= 1 && temp_every < (1ll << 31));
+  if (dist_bias.numel() == 0) return 0;
+  KAITO_CHECK_F32(dist_bias);
+  TORCH_CHECK(dist_bias.dim() == 2 && dist_bias.size(0) == q.size(1) &&
+              dist_bias.size(1) < (1ll << 30),
+              "distance bias: [heads, distances]");
+  TORCH_CHECK(sig_bias.numel() == 0, "distance bias: softmax weights only");
+  return (int)dist_bias.size(1);
 }
 
 }  // namespace
@@ -988,7 +1041,8 @@ void window_attention(at::Tensor out, at::Tensor q, at::Tensor k_cache,
                       double scale, double softcap, at::Tensor r1,
                       at::Tensor r2, int64_t window, int64_t keep_first,
                       at::Tensor sinks, int64_t chunk, at::Tensor sig_bias,
-                      at::Tensor gate) {
+                      at::Tensor gate, at::Tensor dist_bias,
+                      double temp_coef, int64_t temp_every) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() &&
               is_act_dtype(q));
   TORCH_CHECK(keep_first >= 0 && keep_first < (1 << 30));
@@ -1003,6 +1057,9 @@ void window_attention(at::Tensor out, at::Tensor q, at::Tensor k_cache,
     TORCH_CHECK(sinks.numel() == q.size(1));
   }
   check_weights_and_gate(q, sinks, sig_bias, gate);
+  const int db_n = check_distance_bias(q, dist_bias, sig_bias, temp_coef,
+                                       temp_every);
+  const float* db = db_n > 0 ? dist_bias.data_ptr<float>() : nullptr;
   const float* pb = sig_bias.numel() > 0 ? sig_bias.data_ptr<float>()
                                          : nullptr;
   const bool gated = gate.numel() > 0;
@@ -1052,22 +1109,26 @@ void window_attention(at::Tensor out, at::Tensor q, at::Tensor k_cache,
         launch_decode<act_t, 8>(nch, grid, lds_bytes, stream0, out, q,
             k_cache, v_cache, block_tables, token_seq, positions,
             (float)scale, (float)softcap, p1, p2, (int)window, H, G, D, V,
-            BS, KT, kf, ps, (int)chunk, pb, pg, gs0);
+            BS, KT, kf, ps, (int)chunk, pb, pg, gs0, db, db_n,
+            (float)temp_coef, (int)temp_every);
       else if (rt == 4)
         launch_decode<act_t, 4>(nch, grid, lds_bytes, stream0, out, q,
             k_cache, v_cache, block_tables, token_seq, positions,
             (float)scale, (float)softcap, p1, p2, (int)window, H, G, D, V,
-            BS, KT, kf, ps, (int)chunk, pb, pg, gs0);
+            BS, KT, kf, ps, (int)chunk, pb, pg, gs0, db, db_n,
+            (float)temp_coef, (int)temp_every);
       else if (rt == 2)
         launch_decode<act_t, 2>(nch, grid, lds_bytes, stream0, out, q,
             k_cache, v_cache, block_tables, token_seq, positions,
             (float)scale, (float)softcap, p1, p2, (int)window, H, G, D, V,
-            BS, KT, kf, ps, (int)chunk, pb, pg, gs0);
+            BS, KT, kf, ps, (int)chunk, pb, pg, gs0, db, db_n,
+            (float)temp_coef, (int)temp_every);
       else
         launch_decode<act_t, 1>(nch, grid, lds_bytes, stream0, out, q,
             k_cache, v_cache, block_tables, token_seq, positions,
             (float)scale, (float)softcap, p1, p2, (int)window, H, G, D, V,
-            BS, KT, kf, ps, (int)chunk, pb, pg, gs0);
+            BS, KT, kf, ps, (int)chunk, pb, pg, gs0, db, db_n,
+            (float)temp_coef, (int)temp_every);
     });
     return;
   }
@@ -1091,7 +1152,8 @@ void window_attention(at::Tensor out, at::Tensor q, at::Tensor k_cache,
         bias ? r2.data_ptr<float>() : nullptr, (int)window, H, G, D, V, BS,
         kf, has_sinks ? sinks.data_ptr<float>() : nullptr, (int)chunk, pb,
         gated ? (const act_t*)gate.data_ptr() : nullptr,
-        gated ? gate.stride(0) : 0);
+        gated ? gate.stride(0) : 0, db, db_n, (float)temp_coef,
+        (int)temp_every);
   });
 }
 
@@ -1106,7 +1168,9 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
                             double scale, double softcap, at::Tensor r1,
                             at::Tensor r2, int64_t window, int64_t keep_first,
                             at::Tensor sinks, int64_t chunk,
-                            at::Tensor sig_bias, at::Tensor gate) {
+                            at::Tensor sig_bias, at::Tensor gate,
+                            at::Tensor dist_bias, double temp_coef,
+                            int64_t temp_every) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() &&
               q.dtype() == at::kBFloat16);
   TORCH_CHECK(keep_first >= 0 && keep_first < (1 << 30));
@@ -1119,6 +1183,9 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
     TORCH_CHECK(sinks.numel() == q.size(1));
   }
   check_weights_and_gate(q, sinks, sig_bias, gate);
+  const int db_n = check_distance_bias(q, dist_bias, sig_bias, temp_coef,
+                                       temp_every);
+  const float* db = db_n > 0 ? dist_bias.data_ptr<float>() : nullptr;
   const float* pb = sig_bias.numel() > 0 ? sig_bias.data_ptr<float>()
                                          : nullptr;
   const bool gated = gate.numel() > 0;
@@ -1144,11 +1211,13 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
     KAITO_CHECK_F32(r1); KAITO_CHECK_F32(r2);
     TORCH_CHECK(r1.numel() == H && r2.numel() == H);
   }
+  TORCH_CHECK(db_n > 0 || temp_coef == 0.0,
+              "the query temperature comes with a distance bias");
   const int ntiles = tile_seq.size(0);
   if (ntiles == 0 || T == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
-#define KAITO_WIN_LAUNCH(D_, DV_, SIG_)                                      \
-    hipLaunchKernelGGL((window_attention_mfma_kernel<D_, DV_, SIG_>),        \
+#define KAITO_WIN_LAUNCH(D_, DV_, SIG_, DB_)                                 \
+    hipLaunchKernelGGL((window_attention_mfma_kernel<D_, DV_, SIG_, DB_>),   \
         dim3(ntiles, H), dim3(256), 0, stream, (short*)out.data_ptr(),       \
         (const short*)q.data_ptr(), (const short*)k_cache.data_ptr(),        \
         (const short*)v_cache.data_ptr(), tile_seq.data_ptr<int>(),          \
@@ -1159,11 +1228,13 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
         bias ? r2.data_ptr<float>() : nullptr, (int)window, H, G, BS, kf,    \
         has_sinks ? sinks.data_ptr<float>() : nullptr, (int)chunk, pb,       \
         gated ? (const short*)gate.data_ptr() : nullptr,                     \
-        gated ? gate.stride(0) : 0)
+        gated ? gate.stride(0) : 0, db, db_n, (float)temp_coef,              \
+        (int)temp_every)
 #define KAITO_WIN_CASE(D_, DV_)                                              \
   if (D == D_ && V == DV_) {                                                 \
-    if (pb) KAITO_WIN_LAUNCH(D_, DV_, true);                                 \
-    else KAITO_WIN_LAUNCH(D_, DV_, false);                                   \
+    if (pb) KAITO_WIN_LAUNCH(D_, DV_, true, false);                          \
+    else if (db) KAITO_WIN_LAUNCH(D_, DV_, false, true);                     \
+    else KAITO_WIN_LAUNCH(D_, DV_, false, false);                            \
     return;                                                                  \
   }
   KAITO_WIN_CASE(64, 64) KAITO_WIN_CASE(64, 128) KAITO_WIN_CASE(128, 64)
@@ -1179,9 +1250,9 @@ void window_attention_tiles(at::Tensor out, at::Tensor q, at::Tensor k_cache,
 }  // namespace kaito
 
 TORCH_LIBRARY_FRAGMENT(kaito, m) {
-  m.def("window_attention_tiles(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tile_seq, Tensor tile_qbase, Tensor cu_seqlens, Tensor seq_starts, float scale, float softcap, Tensor r1, Tensor r2, int window, int keep_first, Tensor sinks, int chunk, Tensor sig_bias, Tensor gate) -> ()");
+  m.def("window_attention_tiles(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tile_seq, Tensor tile_qbase, Tensor cu_seqlens, Tensor seq_starts, float scale, float softcap, Tensor r1, Tensor r2, int window, int keep_first, Tensor sinks, int chunk, Tensor sig_bias, Tensor gate, Tensor dist_bias, float temp_coef, int temp_every) -> ()");
   m.def("qk_norm_cache_write(Tensor(a!) q_out, Tensor q, Tensor k, Tensor v, Tensor q_w, Tensor k_w, float eps, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slot_mapping, Tensor positions, Tensor inv_freq, float rot_mag, Tensor v_first, float v_lambda, bool unit_norm, bool interleaved) -> ()");
-  m.def("window_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor token_seq, Tensor positions, float scale, float softcap, Tensor r1, Tensor r2, int window, int keep_first, Tensor sinks, int chunk, Tensor sig_bias, Tensor gate) -> ()");
+  m.def("window_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor token_seq, Tensor positions, float scale, float softcap, Tensor r1, Tensor r2, int window, int keep_first, Tensor sinks, int chunk, Tensor sig_bias, Tensor gate, Tensor dist_bias, float temp_coef, int temp_every) -> ()");
 }
 TORCH_LIBRARY_IMPL(kaito, CUDA, m) {
   m.impl("qk_norm_cache_write", &kaito::qk_norm_cache_write);

@@ -6,6 +6,8 @@ kernels against these fp32 references).
 """
 from __future__ import annotations
 
+import math
+
 import torch
 
 
@@ -402,7 +404,8 @@ def qk_norm_cache_write(q, k, v, q_w, k_w, eps: float, k_cache, v_cache,
 def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
                      scale: float, softcap: float, r1, r2, window: int,
                      keep_first: int = 0, sinks=None, chunk: int = 0,
-                     sigmoid_bias=None, gate=None):
+                     sigmoid_bias=None, gate=None, dist_bias=None,
+                     temp_coef: float = 0.0, temp_every: int = 1):
     """Causal sliding-window attention of query rows over the paged cache.
     Row t belongs to chunk token_seq[t] (its block table row) at sequence
     position positions[t] and sees keys j <= pos with pos - j < window or
@@ -411,7 +414,10 @@ def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
     softmax denominator also holds exp(sink_h). With `chunk` > 0 the mask
     is chunked instead: keys j <= pos in pos's block of `chunk` positions
     counted from 0. With `sigmoid_bias` [H] a key's weight is sigmoid(score
-    + bias), not normalised. `gate` [T, H]: outputs times sigmoid(gate)."""
+    + bias), not normalised. `gate` [T, H]: outputs times sigmoid(gate).
+    `dist_bias` [H, N]: its entry min(pos - j, N - 1) joins the score;
+    `temp_coef`: products scaled by 1 + temp_coef*ln((pos + 1) //
+    temp_every + 1)."""
     T, H, D = q.shape
     G, bs, V = k_cache.size(1), k_cache.size(2), v_cache.size(3)
     rep = H // G
@@ -432,12 +438,17 @@ def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
         kk = kk.repeat_interleave(rep, 1)
         vv = vv.repeat_interleave(rep, 1)
         s = torch.einsum("hd,nhd->hn", q[t].float(), kk) * scale
+        if temp_coef != 0:
+            s = s * (1.0 + temp_coef * math.log((p + 1) // temp_every + 1))
         if softcap > 0:
             s = softcap * torch.tanh(s / softcap)
         if r1 is not None:
             dist = (p - js).float()
             s = s - r1.float()[:, None] * torch.log1p(
                 r2.float()[:, None] * dist[None, :])
+        if dist_bias is not None:
+            s = s + dist_bias.float()[
+                :, (p - js).clamp(max=dist_bias.size(1) - 1)]
         if sigmoid_bias is not None:
             w = torch.sigmoid(s + sigmoid_bias.float()[:, None])
         elif sinks is not None:
@@ -661,12 +672,13 @@ def latent_rope_cache_write(q, dkv, norm_w, eps: float, cache, slot_mapping,
 
 
 def latent_attention(q, cache, block_tables, token_seq, positions,
-                     scale: float, rank: int, sinks=None):
+                     scale: float, rank: int, sinks=None, window: int = 0):
     """Causal attention in the latent space. q [T, H, rank + P] (the
     unrotated query already folded through the key up-projection), cache
     [blocks, block_size, rank + P]; row t belongs to chunk token_seq[t]
     (its block-table row; negative: padding) at position positions[t] and
-    sees cached rows 0..position. score = q . row * scale; with `sinks`
+    sees cached rows 0..position (with window > 0 the last `window` of
+    them). score = q . row * scale; with `sinks`
     [H] the softmax denominator also holds exp(sink_h). Returns the
     weighted sum of the rows' first `rank` dims, [T, H, rank]."""
     T, H, DT = q.shape
@@ -677,7 +689,8 @@ def latent_attention(q, cache, block_tables, token_seq, positions,
     for t in range(T):
         if seq_l[t] < 0:
             continue
-        js = torch.arange(pos_l[t] + 1)
+        lo = max(0, pos_l[t] - window + 1) if window > 0 else 0
+        js = torch.arange(lo, pos_l[t] + 1)
         rows = flat[block_tables[seq_l[t]].long()[js // bs] * bs + js % bs]
         rows = rows.float()
         s = q[t].float() @ rows.t() * scale              # [H, n]
@@ -790,7 +803,7 @@ def moe_route(logits, correction, top: int, n_real: int, groups: int,
     n_real)."""
     T, N = logits.shape
     s = torch.softmax(logits.float(), -1)
-    choice = s + correction.float()
+    choice = s if correction is None else s + correction.float()
     if groups > 1:
         best = choice.view(T, groups, -1).amax(-1).topk(keep, -1)[1]
         ok = torch.zeros(T, groups, dtype=torch.bool, device=logits.device)
@@ -842,3 +855,59 @@ def stream_mix_norm(x, y, mix, w_out, w_in, w, eps: float, out_dtype,
     u = (new * w_in.float()[None, :, None]).sum(1)
     return u.to(out_dtype) if w is None else _stream_norm(u, w, eps,
                                                           out_dtype)
+
+
+# ---- sandwich-normed stacks ---------------------------------------------------
+
+def layer_norm_cast(x, w, b, eps: float, out_dtype):
+    xf = x.float()
+    c = xf - xf.mean(-1, keepdim=True)
+    return (c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps)
+            * w.float() + b.float()).to(out_dtype)
+
+
+def embed_layer_norm(ids, table, scale: float, w, b, eps: float):
+    x = table[ids].float() * scale
+    return x, layer_norm_cast(x, w, b, eps, table.dtype)
+
+
+def sandwich_norm_residual(x32, y, w, b, w_next, b_next, eps: float,
+                           out_dtype, y2=None):
+    """x32 += ln(y + y2)*w + b in place; ln(x32)*w_next + b_next in
+    out_dtype (None when w_next is None)."""
+    m = y.float() if y2 is None else y.float() + y2.float()
+    x32 += layer_norm_cast(m, w, b, eps, torch.float32)
+    return None if w_next is None else layer_norm_cast(x32, w_next, b_next,
+                                                       eps, out_dtype)
+
+
+def gla_scan(q, k, v, gate, low, a2, a_bias, tau: float, q_scale: float,
+             norm_w, state, cu_seqlens, state_slots, seq_starts,
+             norm_eps: float):
+    """q/k [T, H, D], v/gate [T, H, V], low [T, R] f32, a2 [R, H*D] f32,
+    a_bias [H*D] f32; state [slots, H, D, V] f32 in place. alpha =
+    sigmoid(low @ a2 + a_bias)^(1/tau); S <- diag(alpha) S + k v^T, o =
+    S^T q * q_scale, RMS-normed over V with norm_w [V], times silu(gate).
+    Returns [T, H*V]."""
+    T, H, D = q.shape
+    V = v.size(2)
+    z = low.float() @ a2.float() + a_bias.float()
+    alpha = torch.exp(torch.nn.functional.logsigmoid(z) / tau).view(T, H, D)
+    qf, kf, vf = q.float() * q_scale, k.float(), v.float()
+    out = torch.zeros(T, H, V)
+    for r0, r1, slot, start in _chunks(cu_seqlens, state_slots, seq_starts):
+        S = state[slot].clone() if start > 0 else torch.zeros(H, D, V)
+        for t in range(r0, r1):
+            S = alpha[t][..., None] * S + kf[t][..., None] * vf[t][:, None]
+            out[t] = torch.einsum("hdv,hd->hv", S, qf[t])
+        state[slot] = S
+    out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + norm_eps) \
+        * norm_w.float() * torch.nn.functional.silu(gate.float())
+    return out.reshape(T, H * V).to(q.dtype)
+
+
+def scaled_softcap(x, scale: float, cap: float):
+    x *= scale
+    if cap > 0:
+        x.copy_(cap * torch.tanh(x / cap))
+    return x
