@@ -61,7 +61,7 @@ def parse_args():
                         "kaito_amd.engine.hybrid_bench.SIZES (default all), "
                         "one JSON line per size and model; --hybrid-models "
                         "picks from gurapel, pokulorn, swa-moe, munerax, lokedra, "
-                        "vemenex, "
+                        "vemenex, labirax, "
                         "mla-moe (the latent-attention MoE transformer)")
     p.add_argument("--hybrid-batch", type=int, default=32)
     p.add_argument("--hybrid-prompt", type=int, default=2048)

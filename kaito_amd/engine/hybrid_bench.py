@@ -1,5 +1,5 @@
 """Prefill and decode throughput of the hybrid stacks (Gurapel, Pokulorn,
-Munerax, Lokedra, Vemenex) beside each other and beside the engine's closest homogeneous
+Munerax, Lokedra, Vemenex, Labirax) beside each other and beside the engine's closest homogeneous
 model at equal size: a sliding-window GQA transformer with the same MoE
 feed-forward (the gpt-oss class without sinks) for the recurrent hybrids
 and Vemenex, the latent-attention MoE transformer (deepseek class) for Munerax. Random
@@ -207,6 +207,45 @@ def vemenex_config(name: str, z: dict, max_pos: int):
         "vocab": z["vocab"], "width": z["width"]}, name=f"vemenex-{name}")
 
 
+def labirax_config(name: str, z: dict, max_pos: int):
+    """The sandwich-normed stack at the sizes of `z`: three layers (gated
+    linear attention, windowed latent attention, attention over every key
+    with a distance bias), then the same three on shared weights, so as many
+    layer runs as the other stacks have layers. Recurrent states match the
+    Gurapel stack's (one dim x dim matrix per head), the latent layer has the
+    Munerax head layout, the window is the other stacks', the experts are the
+    same count and width and a shared expert of that width joins them."""
+    from ..models.hybrid_config import labirax_model_config
+    a = LATENT
+    moe = {"kind": "moe", "expert": {"ff": z["ff"]},
+           "router": {"experts": z["experts"], "top": z["top"]},
+           "shared": {"ff": z["ff"]}}
+    layers = [
+        {"type": "gla", "mlp": moe, "mixer": {
+            "heads": z["heads"], "dim": z["dim"], "vdim": z["dim"],
+            "tau": 16.0}},
+        {"type": "latent_attention", "mlp": moe, "mixer": {
+            "heads": z["heads"], "dim": a["dim"], "rot_dim": a["rot_dim"],
+            "vdim": a["vdim"], "kv_rank": a["kv_rank"],
+            "q_rank": 3 * a["kv_rank"] // 2, "mask": {"size": z["window"]},
+            "scale": (a["dim"] + a["rot_dim"]) ** -0.5,
+            "rot": {"base": 10000.0, "dims": a["rot_dim"]}}},
+        {"type": "attention", "mlp": moe, "mixer": {
+            "heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"],
+            "vdim": z["dim"], "bias_max": z["window"],
+            "scale": z["dim"] ** -0.5,
+            "q_temp": {"coef": 0.1, "every": z["window"]}}},
+    ]
+    return labirax_model_config({
+        "architecture": "Labirax", "embedding": {"scale": 1.0},
+        "layers": [layers[i] if i < 3 else
+                   dict(layers[i % 3], weights_of=i % 3)
+                   for i in range(z["layers"])],
+        "logit_scale": 1.0, "logit_softcap": 30.0,
+        "max_positions": max_pos, "norm": {"eps": 1e-5},
+        "vocab": z["vocab"], "width": z["width"]}, name=f"labirax-{name}")
+
+
 def latent_transformer_config(name: str, z: dict, max_pos: int):
     """The engine's latent-attention MoE transformer (deepseek class) with
     the same head layout, latent rank, experts, groups and shared
@@ -287,6 +326,7 @@ def run(sizes: List[str], batch: int, prompt: int, out_tokens: int,
                     "munerax": munerax_config,
                     "lokedra": lokedra_config,
                     "vemenex": vemenex_config,
+                    "labirax": labirax_config,
                     "mla-moe": latent_transformer_config}[kind](
                         name, z, max_pos)
             pre, dec = _measure(mcfg, batch, prompt, out_tokens, eager)

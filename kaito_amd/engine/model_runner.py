@@ -237,7 +237,7 @@ class ModelRunner:
                 # kernel (a step of single tokens keeps the decode kernel)
                 from .. import ops
                 meta.tile_seq, meta.tile_qbase = ops.build_query_tiles(
-                    [c.length for c in chunks], dev)
+                    [c.length for c in chunks], dev, meta.ctx_starts)
         if self.lora_manager is not None:
             tok_ids = []
             for c in chunks:

@@ -571,14 +571,15 @@ def window_attention(q, k_cache, v_cache, block_tables, token_seq, positions,
                                       temp_coef, temp_every)
 
 
-def build_query_tiles(chunk_lens, device):
+def build_query_tiles(chunk_lens, device, starts=None):
     """Host-side tiling of a step's chunks into 64-row query tiles:
-    (tile_seq, tile_qbase) int32 tensors."""
-    seqs, bases = [], []
-    for i, n in enumerate(chunk_lens):
-        for q0 in range(0, n, QTILE):
-            seqs.append(i)
-            bases.append(q0)
+    (tile_seq, tile_qbase) int32 tensors. Tiles with the most keys ahead
+    of them (`starts`: the chunks' first positions) come first, so that a
+    causal launch does not end on its longest workgroups."""
+    tiles = [(i, q0) for i, n in enumerate(chunk_lens)
+             for q0 in range(0, n, QTILE)]
+    tiles.sort(key=lambda t: -(t[1] + (starts[t[0]] if starts else 0)))
+    seqs, bases = [t[0] for t in tiles], [t[1] for t in tiles]
     return (torch.tensor(seqs, dtype=torch.int32, device=device),
             torch.tensor(bases, dtype=torch.int32, device=device))
 

@@ -131,9 +131,10 @@ KAITO_DEV float log_sigmoid_f(float z) {
   return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
 }
 
-// One wave per (TB tokens, head): a row of A2 is loaded once for all of
-// them. scratch rows: rd (= q*alpha), d (= alpha), k; scalar rk = q.k
-template <typename T, int TB>
+// One wave per (TB tokens, head); lane i holds channels i, i + 64, ... (NI of
+// them). A value of A2 is loaded once for all tokens, four rows at a time.
+// scratch rows: rd (= q*alpha), d (= alpha), k; scalar rk = q.k
+template <typename T, int TB, int NI>
 __global__ __launch_bounds__(64) void gla_prep_kernel(
     float* __restrict__ srd, float* __restrict__ sd, float* __restrict__ sk,
     float* __restrict__ srk,
@@ -144,47 +145,61 @@ __global__ __launch_bounds__(64) void gla_prep_kernel(
     const float* __restrict__ a_bias, const float inv_tau,
     const float q_scale, const int rank, const int NT, const int H,
     const int D, const int DPAD) {
+  constexpr int RU = 4;
   const int t0 = blockIdx.x * TB, h = blockIdx.y, lane = threadIdx.x;
   const int64_t hd = (int64_t)H * D;
-  float rk[TB];
+  float qv[NI][TB], kv[NI][TB], z[NI][TB];
 #pragma unroll
-  for (int u = 0; u < TB; u++) rk[u] = 0.f;
-  for (int i = lane; i < DPAD; i += 64) {
-    const bool in = i < D;
-    float z[TB];
-    if (in) {
-      const float* col = a2 + (int64_t)h * D + i;
-      const float bias = a_bias[(int64_t)h * D + i];
-#pragma unroll
-      for (int u = 0; u < TB; u++) z[u] = bias;
-      for (int r = 0; r < rank; r++) {
-        const float w = col[r * hd];
-#pragma unroll
-        for (int u = 0; u < TB; u++)
-          z[u] += low[(int64_t)min(t0 + u, NT - 1) * low_s0 + r] * w;
-      }
-    }
+  for (int n = 0; n < NI; n++) {
+    const int c = min(lane + 64 * n, D - 1);
+    const float bias = a_bias[(int64_t)h * D + c];
 #pragma unroll
     for (int u = 0; u < TB; u++) {
-      const int t = t0 + u;
-      if (t >= NT) break;
-      float rd = 0.f, d = 0.f, kv = 0.f;
-      if (in) {
-        d = expf(log_sigmoid_f(z[u]) * inv_tau);
-        kv = act_ld(k + (int64_t)t * k_s0 + (int64_t)h * k_s1 + i);
-        const float qv =
-            act_ld(q + (int64_t)t * q_s0 + (int64_t)h * q_s1 + i) * q_scale;
-        rd = qv * d;
-        rk[u] += qv * kv;
+      const int64_t t = min(t0 + u, NT - 1);
+      qv[n][u] = act_ld(q + t * q_s0 + (int64_t)h * q_s1 + c);
+      kv[n][u] = act_ld(k + t * k_s0 + (int64_t)h * k_s1 + c);
+      z[n][u] = bias;
+    }
+  }
+  for (int r0 = 0; r0 < rank; r0 += RU) {
+    float w[NI][RU];
+#pragma unroll
+    for (int j = 0; j < RU; j++)
+#pragma unroll
+      for (int n = 0; n < NI; n++)
+        w[n][j] = r0 + j < rank
+            ? a2[(r0 + j) * hd + (int64_t)h * D + min(lane + 64 * n, D - 1)]
+            : 0.f;
+#pragma unroll
+    for (int u = 0; u < TB; u++) {
+      const float* lr = low + (int64_t)min(t0 + u, NT - 1) * low_s0;
+#pragma unroll
+      for (int j = 0; j < RU; j++) {
+        const float l = lr[min(r0 + j, rank - 1)];
+#pragma unroll
+        for (int n = 0; n < NI; n++) z[n][u] += l * w[n][j];
       }
-      const int64_t o = ((int64_t)t * H + h) * DPAD + i;
-      srd[o] = rd; sd[o] = d; sk[o] = kv;
     }
   }
 #pragma unroll
   for (int u = 0; u < TB; u++) {
-    const float v = wave_reduce_sum(rk[u]);
-    if (lane == 0 && t0 + u < NT) srk[(int64_t)(t0 + u) * H + h] = v;
+    const int t = t0 + u;
+    if (t >= NT) break;
+    float rk = 0.f;
+#pragma unroll
+    for (int n = 0; n < NI; n++) {
+      const int i = lane + 64 * n;
+      if (i >= DPAD) continue;
+      const bool in = i < D;
+      const float d = in ? expf(log_sigmoid_f(z[n][u]) * inv_tau) : 0.f;
+      const float kd = in ? kv[n][u] : 0.f;
+      const float qs = in ? qv[n][u] * q_scale : 0.f;
+      rk += qs * kd;
+      const int64_t o = ((int64_t)t * H + h) * DPAD + i;
+      srd[o] = qs * d; sd[o] = d; sk[o] = kd;
+    }
+    rk = wave_reduce_sum(rk);
+    if (lane == 0) srk[(int64_t)t * H + h] = rk;
   }
 }
 
@@ -594,9 +609,9 @@ void gla_scan(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v,
   float* srd = vp, *sd = vp + vs, *sk = vp + 2 * vs;
   float* srk = sca.data_ptr<float>();
   KAITO_DISPATCH_ACT(q, {
-    auto prep = [&](auto tb) {
+    auto prep = [&](auto tb, auto ni) {
       constexpr int TB = decltype(tb)::value;
-      hipLaunchKernelGGL((gla_prep_kernel<act_t, TB>),
+      hipLaunchKernelGGL((gla_prep_kernel<act_t, TB, decltype(ni)::value>),
           dim3((T + TB - 1) / TB, H), dim3(64), 0, stream, srd, sd, sk, srk,
           (const act_t*)q.data_ptr(), q.stride(0), q.stride(1),
           (const act_t*)k.data_ptr(), k.stride(0), k.stride(1),
@@ -604,8 +619,13 @@ void gla_scan(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v,
           a_bias.data_ptr<float>(), (float)(1.0 / tau), (float)q_scale, rank,
           T, H, D, DPAD);
     };
-    if ((int64_t)T * H >= 16384) prep(std::integral_constant<int, 8>{});
-    else prep(std::integral_constant<int, 1>{});
+    auto by_rows = [&](auto tb) {
+      if (DPAD <= 64) prep(tb, std::integral_constant<int, 1>{});
+      else if (DPAD == 128) prep(tb, std::integral_constant<int, 2>{});
+      else prep(tb, std::integral_constant<int, 4>{});
+    };
+    if ((int64_t)T * H >= 16384) by_rows(std::integral_constant<int, 8>{});
+    else by_rows(std::integral_constant<int, 1>{});
     launch_recurrence<act_t, false>(stream, c.B, H, D, V,
         o.data_ptr<float>(), nullptr, srd, sd, nullptr, sk, nullptr, srk,
         (const act_t*)v.data_ptr(), v.stride(0), v.stride(1),

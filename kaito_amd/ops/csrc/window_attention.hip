@@ -498,8 +498,18 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   // key tiles: those that hold kept first tokens, then the window's
   const int first_end =
       min((keep_first + WKV_TILE - 1) / WKV_TILE * WKV_TILE, kv_begin);
-  for (int kv0 = first_end > 0 ? 0 : kv_begin; kv0 < kv_end;
-       kv0 = (kv0 + WKV_TILE == first_end) ? kv_begin : kv0 + WKV_TILE) {
+  auto next_tile = [&](const int kv0) {
+    return kv0 + WKV_TILE == first_end ? kv_begin : kv0 + WKV_TILE;
+  };
+  const int kv_first = first_end > 0 ? 0 : kv_begin;
+  // this thread's entry of a tile's bias, fetched a tile ahead
+  auto tile_bias = [&](const int kv0) {
+    const int dist = q_abs0 + q0 - kv0 + (int)threadIdx.x - (WKV_TILE - 1);
+    return DB && threadIdx.x < WQ_TILE + WKV_TILE - 1
+        ? db[(int64_t)h * db_n + min(max(dist, 0), db_n - 1)] : 0.f;
+  };
+  float bias_nxt = DB ? tile_bias(kv_first) : 0.f;
+  for (int kv0 = kv_first; kv0 < kv_end; kv0 = next_tile(kv0)) {
     for (int i = threadIdx.x; i < WKV_TILE * D / 8; i += 256) {
       const int row = (i * 8) / D;
       const int col = (i * 8) % D;
@@ -520,12 +530,10 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
 #pragma unroll
       for (int j = 0; j < 8; j++) lds_vt[(col + j) * WPAD + row] = vd[j];
     }
-    if (DB && threadIdx.x < WQ_TILE + WKV_TILE - 1) {
-      const int dist = q_abs0 + q0 - kv0 + (int)threadIdx.x - (WKV_TILE - 1);
-      lds_db[threadIdx.x] =
-          db[(int64_t)h * db_n + min(max(dist, 0), db_n - 1)];
-    }
+    if (DB && threadIdx.x < WQ_TILE + WKV_TILE - 1)
+      lds_db[threadIdx.x] = bias_nxt;
     __syncthreads();
+    if (DB) bias_nxt = tile_bias(next_tile(kv0));
 
     f32x4 sfrag[2];
 #pragma unroll

@@ -200,3 +200,153 @@ def forward(cfg, W, tokens, layers_out=None):
     logits = norm(x, "final.norm") @ W["head"].T * float(cfg["logit_scale"])
     cap = float(cfg["logit_softcap"])
     return cap * np.tanh(logits / cap)
+
+
+# ---- configurations and random checkpoints ---------------------------------------
+
+def attention_layer(heads, kv_heads, dim, vdim, bias_max, scale=None,
+                    temp=(0.3, 16), mlp=None):
+    return {"type": "attention", "mlp": mlp, "mixer": {
+        "heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+        "bias_max": bias_max, "scale": dim ** -0.5 if scale is None else scale,
+        "q_temp": {"coef": temp[0], "every": temp[1]}}}
+
+
+def gla_layer(heads, dim, vdim, tau=8.0, mlp=None):
+    return {"type": "gla", "mlp": mlp, "mixer": {
+        "heads": heads, "dim": dim, "vdim": vdim, "tau": tau}}
+
+
+def latent_layer(heads, dim, rot_dim, vdim, kv_rank, q_rank, window,
+                 base=10000.0, scale=None, mlp=None):
+    return {"type": "latent_attention", "mlp": mlp, "mixer": {
+        "heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim,
+        "kv_rank": kv_rank, "q_rank": q_rank, "mask": {"size": window},
+        "rot": {"base": base, "dims": rot_dim},
+        "scale": (dim + rot_dim) ** -0.5 if scale is None else scale}}
+
+
+def moe(experts, top, ff, shared):
+    return {"kind": "moe", "expert": {"ff": ff},
+            "router": {"experts": experts, "top": top},
+            "shared": {"ff": shared}}
+
+
+def again(layers, i):
+    """One more run of layer i on its weights."""
+    return dict(layers[i], weights_of=i)
+
+
+def make_config(layers, width, vocab, eps=1e-5, embed_scale=0.8,
+                logit_scale=1.7, softcap=12.0):
+    return {"architecture": "Labirax", "embedding": {"scale": embed_scale},
+            "layers": layers, "logit_scale": logit_scale,
+            "logit_softcap": softcap, "norm": {"eps": eps}, "vocab": vocab,
+            "width": width}
+
+
+def bf16_round(a):
+    """Values a bfloat16 file can hold, as float64 (the checkpoint is
+    written in bf16, so oracle and engine must start from equal weights)."""
+    import torch
+    return torch.tensor(np.asarray(a), dtype=torch.float32).to(
+        torch.bfloat16).double().numpy()
+
+
+def random_weights(cfg, seed=0, buckets=8, decay_rank=5):
+    rng = np.random.default_rng(seed)
+    width, vocab = int(cfg["width"]), int(cfg["vocab"])
+    W = {}
+
+    def lin(name, out, inn, gain=1.0):
+        W[name] = bf16_round(rng.normal(0, gain / np.sqrt(inn), (out, inn)))
+
+    def vec(name, n, lo=0.6, hi=1.4):
+        W[name] = bf16_round(rng.uniform(lo, hi, n))
+
+    def gauss(name, shape, std, mean=0.0):
+        W[name] = bf16_round(rng.normal(mean, std, shape))
+
+    def norm(name):
+        vec(name, width)
+        gauss(name + ".b", width, 0.3)
+
+    gauss("embed", (vocab, width), 1.2)
+    norm("final.norm")
+    lin("head", vocab, width)
+    for i, layer in enumerate(cfg["layers"]):
+        if layer.get("weights_of") is not None:
+            continue
+        pre, mx, mlp = f"l{i}.", layer["mixer"], layer.get("mlp")
+        mp, kind = pre + "mix.", layer["type"]
+        H = int(mx["heads"])
+        norm(pre + "norm1")
+        norm(pre + "norm1b")
+        if kind == "gla":
+            D, V = int(mx["dim"]), int(mx["vdim"])
+            for n, out in (("q", H * D), ("k", H * D), ("v", H * V),
+                           ("g", H * V)):
+                lin(mp + n, out, width)
+            lin(mp + "a1", decay_rank, width)
+            lin(mp + "a2", H * D, decay_rank, 2.0)
+            gauss(mp + "a2.b", H * D, 1.5, 1.0)
+            vec(mp + "norm", V)
+            lin(mp + "o", width, H * V)
+        elif kind == "latent_attention":
+            D, P, V, R, Q = (int(mx[k]) for k in ("dim", "rot_dim", "vdim",
+                                                  "kv_rank", "q_rank"))
+            lin(mp + "dq", Q, width)
+            vec(mp + "dq.norm", Q)
+            lin(mp + "uq", H * (D + P), Q, 1.5)
+            lin(mp + "dkv", R + P, width)
+            vec(mp + "dkv.norm", R)
+            lin(mp + "uk", H * D, R, 1.5)
+            lin(mp + "uv", H * V, R)
+            lin(mp + "g", H * V, width, 1.5)
+            lin(mp + "o", width, H * V)
+        else:
+            G, D, V = (int(mx[k]) for k in ("kv_heads", "dim", "vdim"))
+            for n, out in (("q", H * D), ("k", G * D), ("v", G * V)):
+                lin(mp + n, out, width)
+                gauss(mp + n + ".b", out, 0.4)
+            gauss(mp + "rel", (buckets, H), 1.0)
+            lin(mp + "o", width, H * V)
+        if mlp is None:
+            continue
+        norm(pre + "norm2")
+        norm(pre + "norm2b")
+        fp = pre + "mlp."
+        ffs = [(f"e{e}", int(mlp["expert"]["ff"]))
+               for e in range(int(mlp["router"]["experts"]))]
+        if mlp.get("shared"):
+            ffs.append(("shared", int(mlp["shared"]["ff"])))
+        for n, ff in ffs:
+            lin(f"{fp}{n}.gate", ff, width, 1.5)
+            lin(f"{fp}{n}.up", ff, width, 1.5)
+            lin(f"{fp}{n}.down", width, ff)
+        lin(fp + "router", int(mlp["router"]["experts"]), width, 3.0)
+    return W
+
+
+def write_checkpoint(folder, cfg, W):
+    """config.json + model.safetensors (bfloat16) as a served folder."""
+    import torch
+    from safetensors.torch import save_file
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    save_file({k: torch.tensor(np.asarray(v), dtype=torch.float32).to(
+        torch.bfloat16).contiguous() for k, v in W.items()},
+        os.path.join(folder, "model.safetensors"))
+    return folder
+
+
+def model_logits(cfg, W, tokens, layers=None):
+    """Logits [T, vocab] as a float64 torch tensor; `layers`, if a list,
+    receives the stream after every layer."""
+    import torch
+    raw = [] if layers is not None else None
+    out = torch.from_numpy(forward(cfg, W, tokens, raw))
+    if layers is not None:
+        layers.extend(torch.from_numpy(x) for x in raw)
+    return out
