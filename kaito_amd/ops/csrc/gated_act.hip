@@ -70,6 +70,29 @@ __global__ void sigmoid_mul_kernel(T* __restrict__ out,
              sigmoid_f(act_ld(gate + (int64_t)t * g_s0 + i / rep)));
 }
 
+// a gate column per column of x, 16 bytes of each per thread
+template <typename T>
+__global__ void sigmoid_mul_vec_kernel(T* __restrict__ out,
+                                       const T* __restrict__ x,
+                                       const int64_t x_s0,
+                                       const T* __restrict__ gate,
+                                       const int64_t g_s0, const int N) {
+  constexpr int VEC = 16 / (int)sizeof(T);
+  const int t = blockIdx.y;
+  const int i = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
+  if (i >= N) return;
+  T xv[VEC], gv[VEC];
+  *reinterpret_cast<float4_t*>(xv) =
+      *reinterpret_cast<const float4_t*>(x + (int64_t)t * x_s0 + i);
+  *reinterpret_cast<float4_t*>(gv) =
+      *reinterpret_cast<const float4_t*>(gate + (int64_t)t * g_s0 + i);
+#pragma unroll
+  for (int e = 0; e < VEC; e++)
+    act_st(xv + e, act_ld(xv + e) * sigmoid_f(act_ld(gv + e)));
+  *reinterpret_cast<float4_t*>(out + (int64_t)t * N + i) =
+      *reinterpret_cast<const float4_t*>(xv);
+}
+
 // mode 0: gelu_tanh(in[i]) * in[F + i]; mode 1: relu(in[i])^2; mode 2:
 // relu(in[i]) * in[F + i]
 KAITO_DEV float unary_glu_f(const int mode, const float a, const float b) {
@@ -195,9 +218,25 @@ void sigmoid_mul(at::Tensor out, at::Tensor x, at::Tensor gate) {
   const int T = x.size(0), N = x.size(1);
   if (T == 0 || N == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
+  const int vec = 16 / (int)x.element_size();
+  const bool wide = gate.size(1) == N && N % vec == 0 &&
+      x.stride(0) % vec == 0 && gate.stride(0) % vec == 0 &&
+      (uintptr_t)x.data_ptr() % 16 == 0 &&
+      (uintptr_t)gate.data_ptr() % 16 == 0 &&
+      (uintptr_t)out.data_ptr() % 16 == 0;
   for (int t0 = 0; t0 < T; t0 += 65535) {
     const int nt = std::min(65535, T - t0);
     KAITO_DISPATCH_ACT(x, {
+      if (wide) {
+        hipLaunchKernelGGL((sigmoid_mul_vec_kernel<act_t>),
+            dim3((N / vec + 255) / 256, nt), dim3(256), 0, stream,
+            (act_t*)out.data_ptr() + (int64_t)t0 * N,
+            (const act_t*)x.data_ptr() + (int64_t)t0 * x.stride(0),
+            x.stride(0),
+            (const act_t*)gate.data_ptr() + (int64_t)t0 * gate.stride(0),
+            gate.stride(0), N);
+        continue;
+      }
       hipLaunchKernelGGL((sigmoid_mul_kernel<act_t>),
           dim3((N + 255) / 256, nt), dim3(256), 0, stream,
           (act_t*)out.data_ptr() + (int64_t)t0 * N,

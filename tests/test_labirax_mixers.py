@@ -663,6 +663,19 @@ def test_gather_skips_pages_behind_the_window():
     assert tables.tolist() == [[0, 0, 0, 1], [2, 3, 0, 0]]
 
 
+@pytest.mark.parametrize("mode", MODES)
+@pytest.mark.parametrize("n,lead", [(48, 8), (40, 3), (2056, 16)])
+def test_value_gate(mode, n, lead):
+    """A gate column per value column, read as a slice of a wider row
+    (aligned and not)."""
+    dev, dt = mode
+    rng = np.random.default_rng(n)
+    xt, x = act(rng.normal(0, 1, (5, n)), mode)
+    gt, g = act(rng.normal(0, 2, (5, n + 24)), mode)
+    got = ops.sigmoid_mul(xt, gt[:, lead:lead + n])
+    close(got, x * L.sigmoid(g[:, lead:lead + n]), dt, bf16=1e-2)
+
+
 # ---- routed feed-forward ---------------------------------------------------------------
 
 @pytest.mark.parametrize("mode", MODES)
