@@ -44,6 +44,10 @@ class ModelRunner:
         # model the unified chunk metadata (no fresh-prompt fast path)
         self.stateful = bool(getattr(self.model, "uses_state_slots", False))
         self.num_state_slots = 0
+        groups = getattr(self.model, "kernel_groups", ())
+        if self.is_gpu and groups:
+            from .. import ops
+            ops.load_extension(*groups)
         self.kv_caches: List[Tuple[torch.Tensor, torch.Tensor]] = []
         self.num_gpu_blocks = 0
         self.max_model_len = cfg.max_model_len or cfg.model.max_position

@@ -54,6 +54,11 @@ class HybridStackBase(nn.Module):
     # metadata, and never the rotary-model prefill fast path
     uses_state_slots = True
 
+    # kernel groups the stack's ops come from; where several are not built
+    # yet, the runner has them compiled side by side instead of one by one
+    # at first use
+    kernel_groups: tuple = ()
+
     def __init__(self, cfg: ModelConfig):
         super().__init__()
         st = get_state()

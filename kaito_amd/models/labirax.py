@@ -94,6 +94,8 @@ class LabiraxLayer(MixerLayerBase):
 
 
 class LabiraxForCausalLM(HybridStackBase):
+    kernel_groups = ("lnorm", "mix", "latent", "diag", "route", "moe", "core")
+
     def __init__(self, cfg: ModelConfig):
         super().__init__(cfg)
         self.embed_tokens = nn.Embedding(cfg.vocab_size, cfg.hidden_size,

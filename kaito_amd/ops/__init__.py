@@ -60,14 +60,14 @@ def extension_available(group: str = "core") -> bool:
 
 
 def load_extension(*groups: str) -> None:
-    """Load (and build, if absent) kernel groups; no arguments = every
-    group except the lazily-loaded newer ones."""
-    for g in (groups or _LEGACY_GROUPS):
-        if g in _LOADED:
-            continue
-        if not so_path(g).exists():
-            from ._build import build
-            build(groups=[g])
+    """Load (and build together, if absent) kernel groups; no arguments =
+    every group except the lazily-loaded newer ones."""
+    todo = [g for g in (groups or _LEGACY_GROUPS) if g not in _LOADED]
+    absent = [g for g in todo if not so_path(g).exists()]
+    if absent:
+        from ._build import build
+        build(groups=absent)
+    for g in todo:
         torch.ops.load_library(str(so_path(g)))
         _LOADED.add(g)
 
