@@ -1,9 +1,9 @@
 """Prefill and decode throughput of the hybrid stacks (Gurapel, Pokulorn,
-Munerax, Lokedra, Vemenex, Labirax) beside each other and beside the engine's closest homogeneous
-model at equal size: a sliding-window GQA transformer with the same MoE
-feed-forward (the gpt-oss class without sinks) for the recurrent hybrids
-and Vemenex, the latent-attention MoE transformer (deepseek class) for Munerax. Random
-weights, synthetic tokens; all models run through the same LLMEngine
+Munerax, Lokedra, Vemenex, Labirax) beside each other and beside the
+engine's closest homogeneous model at equal size: a sliding-window GQA
+transformer with the same MoE feed-forward (the gpt-oss class without
+sinks) for the recurrent hybrids and Vemenex, the latent-attention MoE
+transformer (deepseek class) for Munerax. Random weights, synthetic tokens; all models run through the same LLMEngine
 (scheduler, paged cache, hipGraph decode).
 
 Used by `bench.py --hybrid-compare`; prints one JSON line per
@@ -241,7 +241,7 @@ def labirax_config(name: str, z: dict, max_pos: int):
         "layers": [layers[i] if i < 3 else
                    dict(layers[i % 3], weights_of=i % 3)
                    for i in range(z["layers"])],
-        "logit_scale": 1.0, "logit_softcap": 30.0,
+        "logit_scale": 1.0, "logit_softcap": 25.0,
         "max_positions": max_pos, "norm": {"eps": 1e-5},
         "vocab": z["vocab"], "width": z["width"]}, name=f"labirax-{name}")
 
