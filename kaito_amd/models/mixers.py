@@ -8,8 +8,8 @@ and a gate per head, optionally with a learned distance bias and a query
 temperature), latent attention (one low-rank latent per token in the
 cache, optionally borrowed from an earlier layer, optionally with
 low-rank queries, optionally windowed), the generalized delta rule with
-per-channel decay, and gated linear attention with a tied write gate (HGRN2) or a low-rank decay
-(GLA). Each is a self-contained module parameterised by its spec
+per-channel decay, and gated linear attention with a tied write gate
+(HGRN2) or a low-rank decay (GLA). Each is a self-contained module parameterised by its spec
 (models/hybrid_config.py), so a design picks and combines them freely.
 
 All follow the same calling convention:
